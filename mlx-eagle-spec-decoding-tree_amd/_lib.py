@@ -1,6 +1,7 @@
-"""ctypes binding of libeagle_mi355x.so (declared in include/eagle_mi355x.h).
+"""ctypes binding of libeagle_mi355x.so (declared in include/eagle_mi355x.h) and
+libhybrid_mi355x.so (declared in include/hybrid_mi355x.h).
 
-The library is never built or replaced at import time: a missing library is a
+A library is never built or replaced at import time: a missing library is a
 hard error (there is no CPU or eager fallback).  Build it with
 `python -m mlx_eagle_spec_decoding_tree_amd.build`.
 """
@@ -10,8 +11,10 @@ from ctypes import c_char_p, c_float, c_int, c_int32, c_long, c_longlong, c_size
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libeagle_mi355x.so")
+HYBRID_LIB_PATH = os.path.join(HERE, "libhybrid_mi355x.so")
 
 _lib = None
+_hybrid = None
 
 # name -> (restype, argtypes); must list every symbol the header declares
 SIGNATURES = {
@@ -96,25 +99,91 @@ SIGNATURES = {
 }
 
 
+# dtype, epilogue and form codes of include/hybrid_mi355x.h
+HYB_BF16, HYB_F32 = 0, 1
+HYB_OUT_T, HYB_OUT_F32, HYB_OUT_ADD_F32, HYB_OUT_RELU2, HYB_OUT_TRANSPOSED = range(5)
+HYB_FORM_ROWS, HYB_FORM_SKINNY, HYB_FORM_GEMM = range(3)
+HYB_GLA_CHUNK = 64
+
+
+def _struct(name, *fields):
+    """A ctypes.Structure from (type, "names ...") pairs in declaration order."""
+    flat = [(n, t) for t, names in fields for n in names.split()]
+    return type(name, (ctypes.Structure,), {"_fields_": flat})
+
+
+HybDenseArgs = _struct("HybDenseArgs", (c_void_p, "x w bias out n_dev len_dev norm_w"), (c_long, "ldx ldo"),
+                       (c_int, "dtype M N K epilogue back norm_d form"), (c_float, "eps"))
+HybGlaArgs = _struct("HybGlaArgs", (c_void_p, "x a2 a2_bias z norm_w state out n_dev workspace"),
+                     (c_size_t, "workspace_bytes"), (c_long, "ldx ldo"),
+                     (c_int, "dtype R H dkp dvp rp dv_true off_q off_k off_v off_g off_a"), (c_float, "qscale tau eps"))
+HybLatentDecodeArgs = _struct("HybLatentDecodeArgs", (c_void_p, "q cache uk uv gate out len_dev n_dev workspace"),
+                              (c_size_t, "workspace_bytes"), (c_long, "ldq ldg ldo cap"),
+                              (c_int, "dtype R H dp dvp rank window"), (c_float, "scale"))
+HybWindowArgs = _struct("HybWindowArgs", (c_void_p, "q k vt gate out len_dev n_dev"), (c_long, "ldq ldk ldv ldg ldo"),
+                        (c_int, "dtype R H dp dvp window back"), (c_float, "scale"))
+
+HYBRID_SIGNATURES = {
+    "hyb_status_string": (c_char_p, [c_int]),
+    "hyb_abi_version": (c_int, []),
+    "hyb_embed": (c_int, [c_int, c_void_p, c_void_p, c_float, c_void_p, c_int] + [c_void_p] * 3 + [c_int] * 3 + [c_void_p]),
+    "hyb_norm_rows": (c_int, [c_int] + [c_void_p] * 3 + [c_float] + [c_void_p] * 2 + [c_int] * 3 + [c_void_p]),
+    "hyb_dense_form": (c_int, [c_int] * 5),
+    "hyb_dense": (c_int, [c_void_p] * 2),
+    "hyb_gla_step": (c_int, [c_void_p] * 2),
+    "hyb_gla_chunk_workspace_bytes": (c_size_t, [c_int] * 4),
+    "hyb_gla_chunks": (c_int, [c_void_p] * 2),
+    "hyb_latent_append": (c_int, [c_int, c_void_p, c_long, c_void_p, c_float, c_void_p, c_long] + [c_void_p] * 2
+                          + [c_int] * 3 + [c_void_p]),
+    "hyb_latent_rank_supported": (c_int, [c_int]),
+    "hyb_latent_decode_workspace_bytes": (c_size_t, [c_int] * 4 + [c_long]),
+    "hyb_latent_decode": (c_int, [c_void_p] * 2),
+    "hyb_window_attention": (c_int, [c_void_p] * 2),
+    "hyb_argmax_workspace_bytes": (c_size_t, [c_int]),
+    "hyb_argmax_rows_f32": (c_int, [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_size_t, c_void_p]),
+    "hyb_token_advance": (c_int, [c_void_p] * 4 + [c_int, c_void_p]),
+    "hyb_advance_len": (c_int, [c_void_p] * 2 + [c_int, c_void_p]),
+}
+
+
 class EagleLibraryMissing(RuntimeError):
     pass
+
+
+def _load(path, signatures):
+    if not os.path.exists(path):
+        raise EagleLibraryMissing(
+            f"{path} not found: build the HIP extension first "
+            "(python -m mlx_eagle_spec_decoding_tree_amd.build); there is no fallback path")
+    handle = ctypes.CDLL(path)
+    for name, (res, args) in signatures.items():
+        fn = getattr(handle, name)
+        fn.restype = res
+        fn.argtypes = args
+    return handle
 
 
 def lib():
     """The loaded C-ABI library; raises if it has not been built."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
-            raise EagleLibraryMissing(
-                f"{LIB_PATH} not found: build the HIP extension first "
-                "(python -m mlx_eagle_spec_decoding_tree_amd.build); there is no fallback path")
-        handle = ctypes.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
-            fn = getattr(handle, name)
-            fn.restype = res
-            fn.argtypes = args
-        _lib = handle
+        _lib = _load(LIB_PATH, SIGNATURES)
     return _lib
+
+
+def hybrid():
+    """The library of the unquantised decoder layers; raises if it has not been built."""
+    global _hybrid
+    if _hybrid is None:
+        _hybrid = _load(HYBRID_LIB_PATH, HYBRID_SIGNATURES)
+    return _hybrid
+
+
+def check_hybrid(rc, what):
+    if rc == 0:
+        return
+    msg = f"{what}: {hybrid().hyb_status_string(rc).decode()} (status {rc})"
+    raise (ValueError if rc in (1, 2, 3, 4, 5) else RuntimeError)(msg)
 
 
 def status_string(rc):

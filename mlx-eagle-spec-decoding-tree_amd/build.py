@@ -1,4 +1,5 @@
-"""Build libeagle_mi355x.so (the C-ABI library) in-tree with hipcc for gfx950.
+"""Build the C-ABI libraries in-tree with hipcc for gfx950: libeagle_mi355x.so (quantised decoder,
+tree verification) and libhybrid_mi355x.so (unquantised decoder layers).
 
     python -m mlx_eagle_spec_decoding_tree_amd.build        # or build.build()
 
@@ -20,6 +21,12 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libeagle_mi355x.so")
+
+# library name -> (source directory, path)
+LIBRARIES = {
+    "eagle": (CSRC, LIB),
+    "hybrid": (os.path.join(CSRC, "hybrid"), os.path.join(HERE, "libhybrid_mi355x.so")),
+}
 
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",
@@ -84,19 +91,44 @@ def hipcc():
     raise RuntimeError("hipcc not found; the HIP extension cannot be built")
 
 
-def sources():
-    return sorted(glob.glob(os.path.join(CSRC, "*.hip")))
+def sources(name="eagle"):
+    return sorted(glob.glob(os.path.join(LIBRARIES[name][0], "*.hip")))
 
 
-def build(verbose=False, jobs=8):
-    """Compile every csrc/*.hip to an object (in parallel) and link the library."""
+def build(verbose=False, jobs=8, libraries=None):
+    """Compile every .hip source of the libraries (all of them by default) to an object (in
+    parallel), link each library; returns the path of the last one built (the quantised decoder's
+    by default)."""
+    lib = None
+    for name in libraries or ("hybrid", "eagle"):
+        lib = _build_library(name, verbose, jobs)
+    return lib
+
+
+def build_missing(libraries):
+    """Build those of the libraries that are not there yet.  Processes that start together build
+    once: the first takes the lock, the others wait for it."""
+    import fcntl
+
+    if all(os.path.exists(LIBRARIES[n][1]) for n in libraries):
+        return
+    os.makedirs(os.path.join(HERE, "build"), exist_ok=True)
+    with open(os.path.join(HERE, "build", ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        missing = [n for n in libraries if not os.path.exists(LIBRARIES[n][1])]
+        if missing:
+            build(libraries=missing)
+
+
+def _build_library(name, verbose, jobs):
     cc = hipcc()
-    objdir = os.path.join(HERE, "build")
+    lib = LIBRARIES[name][1]
+    objdir = os.path.join(HERE, "build", name)
     os.makedirs(objdir, exist_ok=True)
     procs = []
     objs = []
     flags = [f for f in FLAGS if f != "-shared"]
-    for src in sources():
+    for src in sources(name):
         obj = os.path.join(objdir, os.path.basename(src) + ".o")
         objs.append(obj)
         cmd = [cc, *flags, "-c", src, "-o", obj]
@@ -123,13 +155,13 @@ def build(verbose=False, jobs=8):
         print(f"[build] {len(report)} kernels, {len(allowed)} on the allowed list use scratch memory")
         for n, (b, why) in sorted(allowed.items()):
             print(f"[build]   {b:4d} B/lane  {why}: {n}")
-    tmp = LIB + ".tmp"
+    tmp = lib + ".tmp"
     cmd = [cc, "--offload-arch=gfx950", "-shared", "-fPIC", "-fno-gpu-rdc", *objs, "-o", tmp]
     r = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT)
     if r.returncode != 0:
         raise RuntimeError("link failed:\n" + r.stdout.decode(errors="replace"))
-    os.replace(tmp, LIB)
-    return LIB
+    os.replace(tmp, lib)
+    return lib
 
 
 if __name__ == "__main__":

@@ -11,6 +11,71 @@ current length from memory instead of from a launch argument.
 import torch
 
 
+class _Length:
+    """Host length of a layer's sequence state, mirrored by a device scalar all layers share."""
+
+    def __init__(self, capacity, len_dev):
+        self.capacity, self.len_dev, self._offset = capacity, len_dev, 0
+
+    @property
+    def offset(self):
+        return self._offset
+
+    @offset.setter
+    def offset(self, value):
+        self._offset = int(value)
+
+    def sync_len(self):
+        self.len_dev.fill_(self._offset)
+
+
+class LatentCache(_Length):
+    """Latent attention: one vector per token, `latents` [capacity, rank].  Layers that attend with
+    another layer's latents hold the same object."""
+
+    def __init__(self, rank, capacity, device, dtype, len_dev):
+        super().__init__(capacity, len_dev)
+        self.latents = torch.zeros((capacity, rank), dtype=dtype, device=device)
+
+    def clear(self):
+        self.offset = 0
+
+
+class RecurrentState(_Length):
+    """State of a linear-attention layer after `offset` tokens, fp32 [heads, key dim, value dim].  It can
+    be cleared but not rewound: the tokens it has absorbed cannot be taken out."""
+
+    def __init__(self, heads, dim, vdim, capacity, device, len_dev):
+        super().__init__(capacity, len_dev)
+        self.state = torch.zeros((heads, dim, vdim), dtype=torch.float32, device=device)
+
+    @property
+    def offset(self):
+        return self._offset
+
+    @offset.setter
+    def offset(self, value):
+        if int(value) < self._offset:
+            raise ValueError("a recurrent state cannot be rewound; clear() it and feed the tokens again")
+        self._offset = int(value)
+
+    def clear(self):
+        self._offset = 0
+        self.state.zero_()
+
+
+class PromptCache(list):
+    """The per-layer caches of one sequence (and the pass objects built on them, `runner`)."""
+    runner = None
+
+    def clear(self):
+        """An empty sequence in the same buffers."""
+        for c in self:
+            c.clear()
+        if self:
+            self[0].sync_len()
+
+
 class KVCache:
     def __init__(self, n_kv_heads, head_dim, capacity, device, len_dev=None):
         self.keys = torch.zeros((1, n_kv_heads, capacity, head_dim), dtype=torch.float16, device=device)
@@ -49,7 +114,10 @@ class KVCache:
 
 
 def make_prompt_cache(model, capacity=4096):
-    """One cache per layer (mlx_eagle.py:518-519); all layers share one device length."""
+    """One cache per layer (mlx_eagle.py:518-519); all layers share one device length.  A model whose
+    layers keep another kind of state makes its own (`make_cache`)."""
+    if hasattr(model, "make_cache"):
+        return model.make_cache(capacity)
     args = model.args
     dev = model.device
     len_dev = torch.zeros(1, dtype=torch.int32, device=dev)

@@ -1,6 +1,7 @@
-"""Reader for MLX-community 4-bit checkpoints on local disk (mlx_utils.py:59-136).
+"""Reader for checkpoints on local disk: MLX-community 4-bit directories (mlx_utils.py:59-136) and,
+through `registry`, the other model families.
 
-A checkpoint directory holds `config.json` and one or more `model*.safetensors` shards
+A 4-bit checkpoint directory holds `config.json` and one or more `model*.safetensors` shards
 (`weight*.safetensors` in older exports).  Quantised linears and the embedding are stored as
 `<name>.weight` (uint32, eight nibbles per word), `<name>.scales`, `<name>.biases` and an
 optional dense `<name>.bias`; `config["quantization"]` gives `group_size` and `bits`.
@@ -58,11 +59,11 @@ def sanitize(weights):
     return {k: v for k, v in weights.items() if "self_attn.rotary_emb.inv_freq" not in k}
 
 
-def load_weights(model_path, device="cpu"):
+def load_weights(model_path, device="cpu", dtype=torch.float16):
     """All tensors of every shard as a flat dict of torch tensors on `device`.  Packed uint32
     words are kept bit for bit (as int32 storage); floating-point tensors that are not fp16
-    (bf16 exports) are converted to fp16, the type the kernels compute in; a value that does not
-    fit fp16 raises ValueError."""
+    (bf16 exports) are converted to fp16, the type the quantised kernels compute in; a value that does
+    not fit fp16 raises ValueError.  dtype=None keeps every tensor as it is stored."""
     from safetensors import safe_open
 
     out = {}
@@ -72,7 +73,7 @@ def load_weights(model_path, device="cpu"):
                 t = f.get_tensor(key)
                 if t.dtype == torch.uint32:
                     t = t.view(torch.int32)
-                elif t.dtype.is_floating_point and t.dtype != torch.float16:
+                elif dtype is not None and t.dtype.is_floating_point and t.dtype != torch.float16:
                     wide = t
                     t = wide.to(torch.float16)
                     # bf16 / fp32 reach beyond fp16's range: refuse rather than carry inf
@@ -108,14 +109,12 @@ def check_quantized(args, weights):
             raise ValueError(f"{name}.weight is not packed uint32")
 
 
-def load_model(model_path, device, model_config=None):
+def load_model(model_path, device, model_config=None, dtype=None):
     """`load_model(model_path)` of the reference (mlx_utils.py:59-136) for a local directory:
-    returns (Model, config)."""
-    from . import llama
+    returns (Model, config).  config.json selects the model family (`registry`); dtype: name of the
+    storage type, None for the one the family is served in."""
+    from . import registry
 
     config = load_config(model_path)
     config.update(model_config or {})
-    args = model_args_from_config(config)
-    weights = load_weights(model_path, device)
-    check_quantized(args, weights)
-    return llama.Model(args, weights, device), config
+    return registry.resolve(config).load(model_path, config, device, dtype), config

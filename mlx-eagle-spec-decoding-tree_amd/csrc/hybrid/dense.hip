@@ -1,0 +1,574 @@
+// Dense layers of a decoder with unquantised weights (bf16 or fp32 storage, fp32 accumulation):
+// embedding, RMS norm, y = x W^T in three forms chosen by the number of rows, row argmax.
+#include "hybrid.h"
+
+#include <math.h>
+
+namespace {
+
+// ------------------------------------------------------------------------------------
+// Embedding: h[r] = table[token] * scale + position_table[len + r], fp32.
+// ------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void embed_kernel(const int32_t* __restrict__ tokens, const T* __restrict__ table,
+                                                    float scale, const T* __restrict__ pos_table, int max_positions,
+                                                    const int32_t* __restrict__ len_dev,
+                                                    const int32_t* __restrict__ n_dev, float* __restrict__ h, int R,
+                                                    int D, int V) {
+  const int r = blockIdx.x;
+  if (r >= hyb_live(n_dev, R)) return;
+  int tok = tokens[r];
+  tok = tok < 0 ? 0 : (tok < V ? tok : V - 1);      // the host refuses such tokens; never read past the table
+  int pos = *len_dev + r;
+  pos = pos < max_positions ? pos : max_positions - 1;
+  for (int d = threadIdx.x * 4; d < D; d += 1024) {
+    f32x4_t v = load4(table + (size_t)tok * D + d) * scale;
+    if (pos_table) v += load4(pos_table + (size_t)pos * D + d);
+    *reinterpret_cast<f32x4_t*>(h + (size_t)r * D + d) = v;
+  }
+}
+
+// ------------------------------------------------------------------------------------
+// RMS norm of fp32 rows, D columns of which the first d_true count (the rest are zero):
+// out = T(x / sqrt(mean(x^2) + eps) * w).  rows: optional row numbers to gather.
+// ------------------------------------------------------------------------------------
+template <int BLOCK>
+__device__ inline float block_sum(float v, float* red) {
+  v = hyb_wave_sum(v);
+  const int wave = threadIdx.x >> 6;
+  if ((threadIdx.x & 63) == 0) red[wave] = v;
+  __syncthreads();
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < BLOCK / 64; ++i) s += red[i];
+  __syncthreads();
+  return s;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ x, const int32_t* __restrict__ rows,
+                                                        const float* __restrict__ w, float eps, T* __restrict__ out,
+                                                        const int32_t* __restrict__ n_dev, int R, int D, int d_true) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  if (r >= hyb_live(n_dev, R)) return;
+  const float* xr = x + (size_t)(rows ? rows[r] : r) * D;
+  float ss = 0.f;
+  for (int d = threadIdx.x * 4; d < D; d += 1024) {
+    const f32x4_t v = load4(xr + d);
+    ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+  }
+  ss = block_sum<256>(ss, red);
+  const float rstd = 1.f / sqrtf(ss / (float)d_true + eps);
+  for (int d = threadIdx.x * 4; d < D; d += 1024)
+    store4<T>(out + (size_t)r * D + d, load4(xr + d) * rstd * load4(w + d));
+}
+
+// ------------------------------------------------------------------------------------
+// y = x W^T.  Epilogues on the fp32 result.
+// ------------------------------------------------------------------------------------
+struct DenseP {
+  const void* x;
+  const void* w;
+  const float* bias;
+  void* out;
+  const int32_t* n_dev;
+  const int32_t* len_dev;
+  const float* norm_w;
+  long ldx, ldo;
+  int M, N, K, epilogue, back, norm_d;
+  float eps;
+};
+
+// first row of x and number of live rows
+__device__ inline int x_window(const DenseP& p, int* row0) {
+  if (!p.len_dev) {
+    *row0 = 0;
+    return hyb_live(p.n_dev, p.M);
+  }
+  const int len = *p.len_dev, n = p.n_dev ? *p.n_dev : p.M;
+  const int r0 = len > p.back ? len - p.back : 0;
+  const int live = n > 0 ? len + n - r0 : 0;
+  *row0 = r0;
+  return live < p.M ? live : p.M;
+}
+
+template <typename T>
+__device__ inline void emit1(const DenseP& p, int m, int n, float v) {
+  if (p.bias) v += p.bias[n];
+  const size_t at = (size_t)m * p.ldo + n;
+  if (p.epilogue == HYB_OUT_F32) {
+    reinterpret_cast<float*>(p.out)[at] = v;
+  } else if (p.epilogue == HYB_OUT_ADD_F32) {
+    reinterpret_cast<float*>(p.out)[at] += v;
+  } else {
+    if (p.epilogue == HYB_OUT_RELU2) {
+      v = fmaxf(v, 0.f);
+      v = v * v;
+    }
+    reinterpret_cast<T*>(p.out)[at] = (T)v;
+  }
+}
+template <typename T>
+__device__ inline void emit4(const DenseP& p, int m, int n, f32x4_t v) {
+  if (p.bias) v += load4(p.bias + n);
+  const size_t at = (size_t)m * p.ldo + n;
+  if (p.epilogue == HYB_OUT_F32) {
+    store4<float>(reinterpret_cast<float*>(p.out) + at, v);
+  } else if (p.epilogue == HYB_OUT_ADD_F32) {
+    float* o = reinterpret_cast<float*>(p.out) + at;
+    store4<float>(o, load4(o) + v);
+  } else {
+    if (p.epilogue == HYB_OUT_RELU2) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float c = fmaxf(v[e], 0.f);
+        v[e] = c * c;
+      }
+    }
+    store4<T>(reinterpret_cast<T*>(p.out) + at, v);
+  }
+}
+
+__device__ inline float dot8(const Frag<bf16_t>& a, const Frag<bf16_t>& b, float c) {
+#pragma unroll
+  for (int e = 0; e < 8; e += 2)
+    c = __builtin_amdgcn_fdot2_f32_bf16(bf16x2_t{a.v[e], a.v[e + 1]}, bf16x2_t{b.v[e], b.v[e + 1]}, c, false);
+  return c;
+}
+__device__ inline float dot8(const Frag<float>& a, const Frag<float>& b, float c) {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) c = fmaf(a.at(e), b.at(e), c);
+  return c;
+}
+
+// Form 1, at most four rows: vector ALU, one wave per RPW weight rows, 512 columns per step, so
+// that a wave reads whole cache lines of one weight row at a time.  With norm_w, x is the fp32
+// residual stream and every workgroup normalises it itself; its first weights are requested before
+// that.
+template <typename T, int MR, int RPW, bool NORM>
+__global__ __launch_bounds__(256) void dense_rows_kernel(DenseP p) {
+  constexpr int U = 4;
+  extern __shared__ __align__(16) unsigned char smem[];
+  T* xs = reinterpret_cast<T*>(smem);             // NORM: [MR][K]
+  __shared__ float red[4];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int n0 = (blockIdx.x * 4 + wave) * RPW;
+  const int live = hyb_live(p.n_dev, p.M);
+  if (live == 0) return;
+  const T* w[RPW];
+#pragma unroll
+  for (int j = 0; j < RPW; ++j)
+    w[j] = reinterpret_cast<const T*>(p.w) + (size_t)(n0 + j < p.N ? n0 + j : p.N - 1) * p.K;
+  Frag<T> wf[RPW][U];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + u * 512 + lane * 8;
+#pragma unroll
+      for (int j = 0; j < RPW; ++j) wf[j][u] = k < p.K ? Frag<T>::load(w[j] + k) : Frag<T>::zero();
+    }
+  };
+  fetch(0);
+  if (NORM) {
+    for (int m = 0; m < MR; ++m) {
+      const float* xr = reinterpret_cast<const float*>(p.x) + (size_t)(m < live ? m : live - 1) * p.ldx;
+      float ss = 0.f;
+      for (int d = threadIdx.x * 4; d < p.K; d += 1024) {
+        const f32x4_t v = load4(xr + d);
+        ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+      }
+      ss = block_sum<256>(ss, red);
+      const float rstd = 1.f / sqrtf(ss / (float)p.norm_d + p.eps);
+      for (int d = threadIdx.x * 4; d < p.K; d += 1024)
+        store4<T>(xs + (size_t)m * p.K + d, load4(xr + d) * rstd * load4(p.norm_w + d));
+    }
+    __syncthreads();
+  }
+  float acc[RPW][MR];
+#pragma unroll
+  for (int j = 0; j < RPW; ++j)
+#pragma unroll
+    for (int m = 0; m < MR; ++m) acc[j][m] = 0.f;
+  for (int k0 = 0; k0 < p.K; k0 += 512 * U) {
+    if (k0) fetch(k0);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + u * 512 + lane * 8;
+      if (k < p.K) {
+#pragma unroll
+        for (int m = 0; m < MR; ++m) {
+          const T* xr = NORM ? xs + (size_t)m * p.K
+                             : reinterpret_cast<const T*>(p.x) + (size_t)(m < live ? m : live - 1) * p.ldx;
+          const Frag<T> xf = Frag<T>::load(xr + k);
+#pragma unroll
+          for (int j = 0; j < RPW; ++j) acc[j][m] = dot8(wf[j][u], xf, acc[j][m]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < RPW; ++j)
+#pragma unroll
+    for (int m = 0; m < MR; ++m) {
+      const float v = hyb_wave_sum(acc[j][m]);
+      if (lane == 0 && n0 + j < p.N && m < live) emit1<T>(p, m, n0 + j, v);
+    }
+}
+
+// Form 2, up to 64 rows: one workgroup of eight waves per 16 weight rows, the waves share K and
+// add their 16 x 16 tiles through LDS.  Weights are read once, x comes from L2.
+template <typename T, int MT>
+__global__ __launch_bounds__(512) void dense_skinny_kernel(DenseP p) {
+  __shared__ f32x4_t red[8][MT][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int col = lane & 15, g = lane >> 4;
+  const int n0 = blockIdx.x * 16;
+  int row0;
+  const int live = x_window(p, &row0);
+  if (live <= 0) return;
+  const T* w = reinterpret_cast<const T*>(p.w) + (size_t)(n0 + col) * p.K + g * 8;
+  const T* x[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    const int m = t * 16 + col;
+    x[t] = reinterpret_cast<const T*>(p.x) + (size_t)(row0 + (m < live ? m : live - 1)) * p.ldx + g * 8;
+  }
+  f32x4_t acc[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k = wave * 64; k < p.K; k += 512) {
+    const Frag<T> w0 = Frag<T>::load(w + k), w1 = Frag<T>::load(w + k + 32);
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      acc[t] = mma(w0, Frag<T>::load(x[t] + k), acc[t]);
+      acc[t] = mma(w1, Frag<T>::load(x[t] + k + 32), acc[t]);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < MT; ++t) red[wave][t][lane] = acc[t];
+  __syncthreads();
+  if (wave < MT) {
+    f32x4_t s = red[0][wave][lane];
+#pragma unroll
+    for (int i = 1; i < 8; ++i) s += red[i][wave][lane];
+    const int m = wave * 16 + col;
+    if (m < live) emit4<T>(p, m, n0 + g * 4, s);
+  }
+}
+
+// Form 3, many rows: BM x BN output block, four waves 2 x 2, 128 bytes of K per step through LDS
+// (double buffered, 16-byte chunks xored with the row so that reads spread over the banks).
+// TRANS: the block is stored transposed, out[n][m].
+template <typename T, int BM, int BN, bool TRANS>
+__global__ __launch_bounds__(256) void dense_gemm_kernel(DenseP p, int tiles_m, int tiles_n) {
+  constexpr int BK = 128 / sizeof(T), EPC = 16 / sizeof(T);
+  constexpr int TM = BM / 32, TN = BN / 32, SUB = BK / 32;
+  __shared__ __align__(16) unsigned char lds[2][(BM + BN) * 128];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int col = lane & 15, g = lane >> 4;
+  // blocks go round robin over the eight XCDs: give each XCD a contiguous run of tiles
+  const int total = tiles_m * tiles_n;
+  int id = blockIdx.x;
+  const int per = total >> 3;
+  if (id < per * 8) id = (id & 7) * per + (id >> 3);
+  const int m0 = (id % tiles_m) * BM, n0 = (id / tiles_m) * BN;
+  int row0;
+  const int live = x_window(p, &row0);
+  if (m0 >= live) return;
+
+  const int chunk = tid & 7, srow = tid >> 3;        // 32 rows per pass of the workgroup
+  const T* xp[TM];
+  const T* wp[TN];
+#pragma unroll
+  for (int i = 0; i < TM; ++i) {
+    const int m = m0 + srow + 32 * i;
+    xp[i] = reinterpret_cast<const T*>(p.x) + (size_t)(row0 + (m < live ? m : live - 1)) * p.ldx + chunk * EPC;
+  }
+#pragma unroll
+  for (int i = 0; i < TN; ++i) {
+    const int n = n0 + srow + 32 * i;
+    wp[i] = reinterpret_cast<const T*>(p.w) + (size_t)(n < p.N ? n : p.N - 1) * p.K + chunk * EPC;
+  }
+  u32x4_t xr[TM], wr[TN];
+  auto fetch = [&](int k) {
+#pragma unroll
+    for (int i = 0; i < TM; ++i) xr[i] = *reinterpret_cast<const u32x4_t*>(xp[i] + k);
+#pragma unroll
+    for (int i = 0; i < TN; ++i) wr[i] = *reinterpret_cast<const u32x4_t*>(wp[i] + k);
+  };
+  const int spos = srow * 128 + ((chunk ^ (srow & 7)) << 4);
+  auto put = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < TM; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][spos + i * 32 * 128]) = xr[i];
+#pragma unroll
+    for (int i = 0; i < TN; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][BM * 128 + spos + i * 32 * 128]) = wr[i];
+  };
+  const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * (BN / 2);
+  auto frag = [&](const unsigned char* base, int row, int s) {
+    const unsigned char* r = base + row * 128;
+    Frag<T> f;
+    if constexpr (sizeof(T) == 2) {
+      f.v = *reinterpret_cast<const bf16x8_t*>(r + (((s * 4 + g) ^ (row & 7)) << 4));
+    } else {
+      f.lo = *reinterpret_cast<const f32x4_t*>(r + (((2 * g) ^ (row & 7)) << 4));
+      f.hi = *reinterpret_cast<const f32x4_t*>(r + (((2 * g + 1) ^ (row & 7)) << 4));
+    }
+    return f;
+  };
+  f32x4_t acc[TM][TN];
+#pragma unroll
+  for (int a = 0; a < TM; ++a)
+#pragma unroll
+    for (int b = 0; b < TN; ++b) acc[a][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+
+  fetch(0);
+  put(0);
+  __syncthreads();
+  int buf = 0;
+  for (int k = 0; k < p.K; k += BK) {
+    const bool more = k + BK < p.K;
+    if (more) fetch(k + BK);
+    const unsigned char* xl = lds[buf];
+    const unsigned char* wl = lds[buf] + BM * 128;
+#pragma unroll
+    for (int s = 0; s < SUB; ++s) {
+      Frag<T> xf[TM], wf[TN];
+#pragma unroll
+      for (int a = 0; a < TM; ++a) xf[a] = frag(xl, wm + a * 16 + col, s);
+#pragma unroll
+      for (int b = 0; b < TN; ++b) wf[b] = frag(wl, wn + b * 16 + col, s);
+#pragma unroll
+      for (int a = 0; a < TM; ++a)
+#pragma unroll
+        for (int b = 0; b < TN; ++b) acc[a][b] = TRANS ? mma(xf[a], wf[b], acc[a][b]) : mma(wf[b], xf[a], acc[a][b]);
+    }
+    if (more) {
+      put(buf ^ 1);
+      __syncthreads();
+      buf ^= 1;
+    }
+  }
+#pragma unroll
+  for (int a = 0; a < TM; ++a)
+#pragma unroll
+    for (int b = 0; b < TN; ++b) {
+      if (TRANS) {
+        const int n = n0 + wn + b * 16 + col, m = m0 + wm + a * 16 + g * 4;
+        // whole groups of four columns: the row of `out` is padded to the block size
+        if (n < p.N && m < live) store4<T>(reinterpret_cast<T*>(p.out) + (size_t)n * p.ldo + m, acc[a][b]);
+      } else {
+        const int m = m0 + wm + a * 16 + col, n = n0 + wn + b * 16 + g * 4;
+        if (n < p.N && m < live) emit4<T>(p, m, n, acc[a][b]);
+      }
+    }
+}
+
+template <typename T, int MR, int RPW>
+void launch_rows(const DenseP& p, bool norm, hipStream_t st) {
+  const int blocks = (p.N + 4 * RPW - 1) / (4 * RPW);
+  if (norm)
+    dense_rows_kernel<T, MR, RPW, true><<<blocks, 256, (size_t)MR * p.K * sizeof(T), st>>>(p);
+  else
+    dense_rows_kernel<T, MR, RPW, false><<<blocks, 256, 0, st>>>(p);
+}
+template <typename T>
+void dense_rows(const DenseP& p, bool norm, hipStream_t st) {
+  const bool wide = p.N >= 16384;                   // enough rows to fill the GPU with two per wave
+  if (p.M == 1)
+    wide ? launch_rows<T, 1, 2>(p, norm, st) : launch_rows<T, 1, 1>(p, norm, st);
+  else if (p.M == 2)
+    wide ? launch_rows<T, 2, 2>(p, norm, st) : launch_rows<T, 2, 1>(p, norm, st);
+  else
+    launch_rows<T, 4, 1>(p, norm, st);
+}
+template <typename T>
+void dense_skinny(const DenseP& p, hipStream_t st) {
+  const int blocks = p.N / 16;
+  if (p.M <= 16)
+    dense_skinny_kernel<T, 1><<<blocks, 512, 0, st>>>(p);
+  else if (p.M <= 32)
+    dense_skinny_kernel<T, 2><<<blocks, 512, 0, st>>>(p);
+  else
+    dense_skinny_kernel<T, 4><<<blocks, 512, 0, st>>>(p);
+}
+template <typename T, int BM, int BN>
+void launch_gemm(const DenseP& p, hipStream_t st) {
+  const int tm = (p.M + BM - 1) / BM, tn = (p.N + BN - 1) / BN;
+  if (p.epilogue == HYB_OUT_TRANSPOSED)
+    dense_gemm_kernel<T, BM, BN, true><<<tm * tn, 256, 0, st>>>(p, tm, tn);
+  else
+    dense_gemm_kernel<T, BM, BN, false><<<tm * tn, 256, 0, st>>>(p, tm, tn);
+}
+template <typename T>
+void dense_gemm(const DenseP& p, hipStream_t st) {
+  auto blocks = [&](int bm, int bn) { return (long)((p.M + bm - 1) / bm) * ((p.N + bn - 1) / bn); };
+  if (blocks(128, 128) >= 256)
+    launch_gemm<T, 128, 128>(p, st);
+  else if (blocks(64, 128) >= 256)
+    launch_gemm<T, 64, 128>(p, st);
+  else
+    launch_gemm<T, 64, 64>(p, st);
+}
+
+// ------------------------------------------------------------------------------------
+// Row argmax of fp32 logits, lowest index among equal maxima.
+// ------------------------------------------------------------------------------------
+struct Best {
+  float v;
+  int i;
+};
+__device__ inline Best better(Best a, Best b) { return (b.v > a.v || (b.v == a.v && b.i < a.i)) ? b : a; }
+__device__ inline Best wave_best(Best b) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    Best c{__shfl_xor(b.v, o, 64), __shfl_xor(b.i, o, 64)};
+    b = better(b, c);
+  }
+  return b;
+}
+constexpr int ARGMAX_PARTS = 64;
+
+__global__ __launch_bounds__(256) void argmax_part_kernel(const float* __restrict__ logits, long ld, int V, float* __restrict__ pv,
+                                                          int32_t* __restrict__ pi) {
+  __shared__ Best red[4];
+  const float* x = logits + (size_t)blockIdx.y * ld;
+  Best b{-INFINITY, 0x7fffffff};
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < V; i += ARGMAX_PARTS * 256) b = better(b, Best{x[i], i});
+  b = wave_best(b);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = b;
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int k = 1; k < 4; ++k) b = better(b, red[k]);
+    pv[blockIdx.y * ARGMAX_PARTS + blockIdx.x] = b.v;
+    pi[blockIdx.y * ARGMAX_PARTS + blockIdx.x] = b.i;
+  }
+}
+__global__ __launch_bounds__(64) void argmax_final_kernel(const float* __restrict__ pv, const int32_t* __restrict__ pi,
+                                                          int32_t* __restrict__ out, int V) {
+  const int at = blockIdx.x * ARGMAX_PARTS + threadIdx.x;
+  const Best b = wave_best(Best{pv[at], pi[at]});
+  if (threadIdx.x == 0) out[blockIdx.x] = b.i < V ? b.i : 0;     // a row of NaN selects token 0
+}
+
+// Loop state after a decoded token: it is appended to the output and becomes the next input.
+__global__ void token_advance_kernel(const int32_t* __restrict__ token, int32_t* __restrict__ next,
+                                     int32_t* __restrict__ out, int32_t* __restrict__ count, int max_out) {
+  const int t = *token, c = *count;
+  *next = t;
+  if (c < max_out) out[c] = t;
+  *count = c + 1;
+}
+__global__ void advance_len_kernel(int32_t* len, const int32_t* n, int capacity) {
+  const int v = *len + (*n > 0 ? *n : 0);
+  *len = v < capacity ? v : capacity;
+}
+
+}  // namespace
+
+HYB_EXPORT int hyb_embed(int dtype, const int32_t* tokens, const void* table, float scale, const void* pos_table,
+                         int max_positions, const int32_t* len_dev, const int32_t* n_dev, float* h, int R, int D, int V,
+                         hyb_stream_t stream) {
+  if (!tokens || !table || !len_dev || !h) return HYB_ERR_NULL;
+  if (dtype != HYB_BF16 && dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (R < 1 || D < 4 || D % 4 || V < 1 || (pos_table && max_positions < 1)) return HYB_ERR_SHAPE;
+  if (!hyb_aligned16(table) || !hyb_aligned16(h)) return HYB_ERR_ALIGN;
+  HYB_DISPATCH(dtype, embed_kernel<T><<<R, 256, 0, (hipStream_t)stream>>>(
+                          tokens, (const T*)table, scale, (const T*)pos_table, pos_table ? max_positions : 0x7fffffff,
+                          len_dev, n_dev, h, R, D, V);)
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_norm_rows(int dtype, const float* x, const int32_t* rows, const float* w, float eps, void* out,
+                             const int32_t* n_dev, int R, int D, int d_true, hyb_stream_t stream) {
+  if (!x || !w || !out) return HYB_ERR_NULL;
+  if (dtype != HYB_BF16 && dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (R < 1 || D < 4 || D % 4 || d_true < 1 || d_true > D) return HYB_ERR_SHAPE;
+  if (!hyb_aligned16(x) || !hyb_aligned16(w) || !hyb_aligned16(out)) return HYB_ERR_ALIGN;
+  HYB_DISPATCH(dtype, norm_rows_kernel<T><<<R, 256, 0, (hipStream_t)stream>>>(x, rows, w, eps, (T*)out, n_dev, R, D,
+                                                                              d_true);)
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_dense_form(int dtype, int M, int K, int norm, int transposed) {
+  const size_t elt = dtype == HYB_BF16 ? 2 : 4;
+  const int mr = M <= 2 ? M : 4;
+  if (!transposed && M <= 4 && (!norm || mr * (size_t)K * elt <= 65536)) return HYB_FORM_ROWS;
+  if (norm) return -1;
+  return !transposed && M <= 64 ? HYB_FORM_SKINNY : HYB_FORM_GEMM;
+}
+
+HYB_EXPORT int hyb_dense(const hyb_dense_args* a, hyb_stream_t stream) {
+  if (!a || !a->x || !a->w || !a->out) return HYB_ERR_NULL;
+  if (a->dtype != HYB_BF16 && a->dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (a->epilogue < HYB_OUT_T || a->epilogue > HYB_OUT_TRANSPOSED) return HYB_ERR_UNSUPPORTED;
+  const bool trans = a->epilogue == HYB_OUT_TRANSPOSED;
+  if (a->M < 1 || a->N < 16 || a->N % 16 || a->K < 64 || a->K % 64) return HYB_ERR_SHAPE;
+  if (a->ldx < a->K || a->ldx % 8 || a->ldo % 4 || a->ldo < (trans ? a->M : a->N)) return HYB_ERR_SHAPE;
+  if (trans && (a->bias || a->ldo % 128)) return HYB_ERR_SHAPE;      // whole blocks of columns are stored
+  if (!hyb_aligned16(a->x) || !hyb_aligned16(a->w) || !hyb_aligned16(a->out) || !hyb_aligned16(a->bias) ||
+      !hyb_aligned16(a->norm_w))
+    return HYB_ERR_ALIGN;
+  if (a->norm_w && (a->norm_d < 1 || a->norm_d > a->K)) return HYB_ERR_SHAPE;
+  int form = hyb_dense_form(a->dtype, a->M, a->K, a->norm_w != nullptr, trans);
+  if (a->form >= 0) {
+    if (a->form > HYB_FORM_GEMM) return HYB_ERR_UNSUPPORTED;
+    if (a->form == HYB_FORM_ROWS && form != HYB_FORM_ROWS) return HYB_ERR_UNSUPPORTED;
+    if (a->form == HYB_FORM_SKINNY && (a->M > 64 || trans || a->norm_w)) return HYB_ERR_UNSUPPORTED;
+    if (a->form == HYB_FORM_GEMM && a->norm_w) return HYB_ERR_UNSUPPORTED;
+    form = a->form;
+  }
+  if (form < 0) return HYB_ERR_UNSUPPORTED;
+  if (a->len_dev && form == HYB_FORM_ROWS) form = HYB_FORM_SKINNY;   // a window of rows: the matrix forms
+  if (a->len_dev && a->norm_w) return HYB_ERR_UNSUPPORTED;
+  DenseP p{a->x,   a->w,   a->bias, a->out, a->n_dev,    a->len_dev, a->norm_w, a->ldx,
+           a->ldo, a->M,   a->N,    a->K,   a->epilogue, a->back,    a->norm_d, a->eps};
+  hipStream_t st = (hipStream_t)stream;
+  HYB_DISPATCH(a->dtype, if (form == HYB_FORM_ROWS) dense_rows<T>(p, a->norm_w != nullptr, st);
+               else if (form == HYB_FORM_SKINNY) dense_skinny<T>(p, st); else dense_gemm<T>(p, st);)
+  return hyb_launch_status();
+}
+
+HYB_EXPORT size_t hyb_argmax_workspace_bytes(int R) { return R < 1 ? 0 : (size_t)R * ARGMAX_PARTS * 8; }
+
+HYB_EXPORT int hyb_argmax_rows_f32(const float* logits, long ld, int R, int V, int32_t* out, void* ws, size_t ws_bytes,
+                                   hyb_stream_t stream) {
+  if (!logits || !out) return HYB_ERR_NULL;
+  if (R < 1 || V < 1 || ld < V) return HYB_ERR_SHAPE;
+  if (!ws || ws_bytes < hyb_argmax_workspace_bytes(R)) return HYB_ERR_WORKSPACE;
+  float* pv = (float*)ws;
+  int32_t* pi = (int32_t*)(pv + (size_t)R * ARGMAX_PARTS);
+  argmax_part_kernel<<<dim3(ARGMAX_PARTS, R), 256, 0, (hipStream_t)stream>>>(logits, ld, V, pv, pi);
+  argmax_final_kernel<<<R, 64, 0, (hipStream_t)stream>>>(pv, pi, out, V);
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_token_advance(const int32_t* token, int32_t* next, int32_t* out, int32_t* count, int max_out,
+                                 hyb_stream_t stream) {
+  if (!token || !next || !out || !count) return HYB_ERR_NULL;
+  if (max_out < 1) return HYB_ERR_SHAPE;
+  token_advance_kernel<<<1, 1, 0, (hipStream_t)stream>>>(token, next, out, count, max_out);
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_advance_len(int32_t* len_dev, const int32_t* n_dev, int capacity, hyb_stream_t stream) {
+  if (!len_dev || !n_dev) return HYB_ERR_NULL;
+  if (capacity < 1) return HYB_ERR_SHAPE;
+  advance_len_kernel<<<1, 1, 0, (hipStream_t)stream>>>(len_dev, n_dev, capacity);
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_abi_version(void) { return 1; }
+
+HYB_EXPORT const char* hyb_status_string(int status) {
+  switch (status) {
+    case HYB_OK: return "ok";
+    case HYB_ERR_NULL: return "required pointer is NULL";
+    case HYB_ERR_SHAPE: return "a dimension is out of the supported range";
+    case HYB_ERR_ALIGN: return "pointer is not 16-byte aligned";
+    case HYB_ERR_UNSUPPORTED: return "form, dtype or epilogue not supported for this shape";
+    case HYB_ERR_WORKSPACE: return "workspace missing or too small";
+    case HYB_ERR_HIP: return "the HIP runtime reported a launch error";
+    default: return "unknown status";
+  }
+}

@@ -1,0 +1,150 @@
+// Shared declarations of the kernels behind include/hybrid_mi355x.h (gfx950): dense layers, gated
+// linear attention and latent attention in bf16 or fp32 storage.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+#include "../../../include/hybrid_mi355x.h"
+
+#define HYB_EXPORT extern "C" __attribute__((visibility("default")))
+
+typedef __bf16 bf16_t;
+typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+typedef __bf16 bf16x4_t __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
+
+static inline bool hyb_aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15u) == 0; }
+static inline int hyb_launch_status() { return hipGetLastError() == hipSuccess ? HYB_OK : HYB_ERR_HIP; }
+
+// Runs `body` with T bound to the storage type of a dtype code.
+#define HYB_DISPATCH(dtype, ...)           \
+  if ((dtype) == HYB_BF16) {               \
+    using T = bf16_t;                      \
+    __VA_ARGS__                            \
+  } else {                                 \
+    using T = float;                       \
+    __VA_ARGS__                            \
+  }
+
+__device__ inline float hyb_wave_sum(float v) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+
+// ------------------------------------------------------------------------------------
+// Eight consecutive elements of a row: the unit of every load and the operand of one matrix
+// step over 32 values of k.  In a 16 x 16 tile lane l holds row (or column) l % 16 and the
+// k values 8 * (l / 16) .. + 7; the result has column l % 16 and rows 4 * (l / 16) .. + 3.
+// The fp32 form issues one 16x16x4 instruction per element, so that k is walked in another
+// order with the same operands: both storage types share every kernel.
+// ------------------------------------------------------------------------------------
+template <typename T>
+struct Frag;
+template <>
+struct Frag<bf16_t> {
+  bf16x8_t v;
+  __device__ static Frag zero() {
+    Frag f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f.v[e] = (bf16_t)0.f;
+    return f;
+  }
+  __device__ static Frag load(const bf16_t* p) {
+    Frag f;
+    f.v = *reinterpret_cast<const bf16x8_t*>(p);
+    return f;
+  }
+  __device__ void store(bf16_t* p) const { *reinterpret_cast<bf16x8_t*>(p) = v; }
+  __device__ float at(int e) const { return (float)v[e]; }
+  __device__ void set(int e, float x) { v[e] = (bf16_t)x; }
+};
+template <>
+struct Frag<float> {
+  f32x4_t lo, hi;
+  __device__ static Frag zero() {
+    Frag f;
+    f.lo = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    f.hi = f.lo;
+    return f;
+  }
+  __device__ static Frag load(const float* p) {
+    Frag f;
+    f.lo = *reinterpret_cast<const f32x4_t*>(p);
+    f.hi = *reinterpret_cast<const f32x4_t*>(p + 4);
+    return f;
+  }
+  __device__ void store(float* p) const {
+    *reinterpret_cast<f32x4_t*>(p) = lo;
+    *reinterpret_cast<f32x4_t*>(p + 4) = hi;
+  }
+  __device__ float at(int e) const { return e < 4 ? lo[e] : hi[e - 4]; }
+  __device__ void set(int e, float x) {
+    if (e < 4)
+      lo[e] = x;
+    else
+      hi[e - 4] = x;
+  }
+};
+
+__device__ inline f32x4_t mma(const Frag<bf16_t>& a, const Frag<bf16_t>& b, f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
+}
+__device__ inline f32x4_t mma(const Frag<float>& a, const Frag<float>& b, f32x4_t c) {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.at(e), b.at(e), c, 0, 0, 0);
+  return c;
+}
+// One operand given in fp32.  bf16 storage: as a sum of two bf16 values (16 significant bits),
+// so that an fp32 intermediate (attention weights, absorbed queries) is not rounded to bf16.
+struct Wide8 {
+  float v[8];
+};
+__device__ inline void split(const Wide8& w, Frag<bf16_t>& hi, Frag<bf16_t>& lo) {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const bf16_t h = (bf16_t)w.v[e];
+    hi.v[e] = h;
+    lo.v[e] = (bf16_t)(w.v[e] - (float)h);
+  }
+}
+__device__ inline Frag<float> as_frag(const Wide8& w) {
+  Frag<float> f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) f.set(e, w.v[e]);
+  return f;
+}
+// c += A B with A fp32 / with B fp32
+__device__ inline f32x4_t mma_wide_a(const Wide8& a, const Frag<bf16_t>& b, f32x4_t c) {
+  Frag<bf16_t> hi, lo;
+  split(a, hi, lo);
+  return mma(hi, b, mma(lo, b, c));
+}
+__device__ inline f32x4_t mma_wide_a(const Wide8& a, const Frag<float>& b, f32x4_t c) { return mma(as_frag(a), b, c); }
+template <typename T>
+__device__ inline void store4(T* p, f32x4_t v);
+template <>
+__device__ inline void store4<float>(float* p, f32x4_t v) {
+  *reinterpret_cast<f32x4_t*>(p) = v;
+}
+template <>
+__device__ inline void store4<bf16_t>(bf16_t* p, f32x4_t v) {
+  *reinterpret_cast<bf16x4_t*>(p) = bf16x4_t{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+}
+__device__ inline f32x4_t load4(const float* p) { return *reinterpret_cast<const f32x4_t*>(p); }
+__device__ inline f32x4_t load4(const bf16_t* p) {
+  const bf16x4_t v = *reinterpret_cast<const bf16x4_t*>(p);
+  return f32x4_t{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+
+__device__ inline float hyb_sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ inline float hyb_log_sigmoid(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
+
+// Rows that really exist among the R a launch is laid out for.
+__device__ inline int hyb_live(const int32_t* n_dev, int R) {
+  if (!n_dev) return R;
+  const int n = *n_dev;
+  return n < 0 ? 0 : (n < R ? n : R);
+}

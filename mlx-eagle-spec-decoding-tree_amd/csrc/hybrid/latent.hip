@@ -1,0 +1,602 @@
+// Latent attention without positions: the cache holds one normed vector c per token, keys and
+// values are W_uk c and W_uv c; causal sliding window, softmax, sigmoid output gate.
+//
+// Few query rows (decoding): the key projection is absorbed into the query (score = (W_uk^T q) . c)
+// and the value projection applied to the weighted sum of c, so that a key costs its cached bytes.
+// Many rows (a prompt portion): keys and values of the visible span are projected once and a
+// windowed attention kernel runs over them.
+#include "hybrid.h"
+
+#include <math.h>
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+// ------------------------------------------------------------------------------------
+// c = norm(W_dkv h) into cache row len + r.  One wave per row.
+// ------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void latent_append_kernel(const T* __restrict__ x, long ldx,
+                                                            const float* __restrict__ w, float eps, T* __restrict__ cache,
+                                                            long cap, const int32_t* __restrict__ len_dev,
+                                                            const int32_t* __restrict__ n_dev, int R, int rank, int rank_true) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (r >= hyb_live(n_dev, R)) return;
+  const long row = (long)*len_dev + r;
+  if (row >= cap) return;                       // the host checks the capacity; never write past it
+  const T* xr = x + (size_t)r * ldx;
+  float ss = 0.f;
+  for (int d = lane * 4; d < rank; d += 256) {
+    const f32x4_t v = load4(xr + d);
+    ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+  }
+  ss = hyb_wave_sum(ss);
+  const float rstd = 1.f / sqrtf(ss / (float)rank_true + eps);
+  for (int d = lane * 4; d < rank; d += 256) store4<T>(cache + (size_t)row * rank + d, load4(xr + d) * rstd * load4(w + d));
+}
+
+// ------------------------------------------------------------------------------------
+// Absorbed queries, fp32: qa[r][h][:] = sum_d q[r][h][d] W_uk[h dp + d][:].
+// Workgroup = one head and 64 latent columns; 32 groups of eight lanes share d.
+// ------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void absorb_kernel(const T* __restrict__ q, long ldq, const T* __restrict__ uk,
+                                                     float* __restrict__ qa, const int32_t* __restrict__ n_dev, int R, int H,
+                                                     int dp, int rank) {
+  __shared__ float red[4][4][64];
+  const int h = blockIdx.x, c0 = blockIdx.y * 64;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int cl = (lane & 7) * 8, dg = wave * 8 + (lane >> 3);
+  const int live = hyb_live(n_dev, R);
+  const T* wk = uk + (size_t)h * dp * rank + c0 + cl;
+  for (int r0 = 0; r0 < live; r0 += 4) {
+    float acc[4][8];
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[r][e] = 0.f;
+    for (int d = dg; d < dp; d += 32) {
+      const Frag<T> w = Frag<T>::load(wk + (size_t)d * rank);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int rr = r0 + r < live ? r0 + r : live - 1;
+        const float qv = (float)q[(size_t)rr * ldq + h * dp + d];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[r][e] = fmaf(qv, w.at(e), acc[r][e]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        float v = acc[r][e];
+        v += __shfl_xor(v, 8, 64);
+        v += __shfl_xor(v, 16, 64);
+        v += __shfl_xor(v, 32, 64);
+        if (lane < 8) red[wave][r][cl + e] = v;
+      }
+    __syncthreads();
+    const int r = threadIdx.x >> 6, c = threadIdx.x & 63;
+    if (r0 + r < live) qa[((size_t)(r0 + r) * H + h) * rank + c0 + c] = red[0][r][c] + red[1][r][c] + red[2][r][c] + red[3][r][c];
+    __syncthreads();
+  }
+}
+
+// ------------------------------------------------------------------------------------
+// Attention of absorbed queries over one split of the keys.  Sixteen query rows (row = r H + h)
+// per workgroup; the cached vectors of 32 keys at a time in LDS.  Partial result per split and
+// row: unnormalised sum of c, maximum and sum of the weights.
+// NCT = rank / 64: column tiles of 16 per wave.
+// ------------------------------------------------------------------------------------
+template <typename T, int NCT>
+__global__ __launch_bounds__(256) void latent_split_kernel(const float* __restrict__ qa, const T* __restrict__ cache,
+                                                           const int32_t* __restrict__ len_dev,
+                                                           const int32_t* __restrict__ n_dev, float* __restrict__ ctx,
+                                                           float* __restrict__ ml, int R, int H, int window, float scale,
+                                                           int keys_per_split, long cap) {
+  constexpr int RANK = NCT * 64;
+  constexpr int LDC = RANK + 16 / sizeof(T);
+  extern __shared__ __align__(16) unsigned char smem[];
+  T* cs = reinterpret_cast<T*>(smem);            // [32][LDC]
+  __shared__ float ss[2][16][33];
+  __shared__ __align__(16) float ps[16][36];
+  __shared__ float al[16];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int col = lane & 15, g = lane >> 4;
+  const int live = hyb_live(n_dev, R), rows = live * H, q0 = blockIdx.x * 16;
+  if (q0 >= rows) return;
+  const int len = *len_dev;
+  const int last = q0 + 15 < rows ? q0 + 15 : rows - 1;
+  const int base = len - window + 1 > 0 ? len - window + 1 : 0;
+  const int first_key = len + q0 / H - window + 1;           // of the first row of this group
+  int lo = base + blockIdx.y * keys_per_split, hi = lo + keys_per_split;      // [lo, hi)
+  lo = lo > first_key ? lo : first_key;
+  const int end = len + last / H + 1;
+  hi = hi < end ? hi : end;
+  hi = hi < cap ? hi : (int)cap;
+  const size_t slot = (size_t)blockIdx.y * R * H;
+  // the row whose softmax this thread helps with: 16 threads per row, two keys each
+  const int srow = threadIdx.x >> 4, sk = threadIdx.x & 15;
+  if (lo >= hi) {
+    if (sk == 0 && q0 + srow < rows) {
+      ml[(slot + q0 + srow) * 2] = -INFINITY;
+      ml[(slot + q0 + srow) * 2 + 1] = 0.f;
+    }
+    return;
+  }
+  const int pos = len + (q0 + srow) / H;
+  const bool real = q0 + srow < rows;
+  const float* qrow = qa + (size_t)(q0 + col < rows ? q0 + col : rows - 1) * RANK + g * 8;
+  f32x4_t acc[NCT];
+#pragma unroll
+  for (int i = 0; i < NCT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+
+  for (int k0 = lo; k0 < hi; k0 += 32) {
+    // stage 32 cached vectors (rows past the end repeat the last one; their weight is zero)
+    for (int i = threadIdx.x; i < 32 * (RANK / 8); i += 256) {
+      const int kr = i / (RANK / 8), c = (i % (RANK / 8)) * 8;
+      const int key = k0 + kr < hi ? k0 + kr : hi - 1;
+      Frag<T>::load(cache + (size_t)key * RANK + c).store(cs + kr * LDC + c);
+    }
+    __syncthreads();
+    {
+      const int kt = wave & 1, half = wave >> 1;             // 16 keys, every second step of 32 columns
+      f32x4_t s = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int st = 0; st < NCT; ++st) {
+        const int c = (2 * st + half) * 32;
+        Wide8 qv;
+        const f32x4_t a = load4(qrow + c), b = load4(qrow + c + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          qv.v[e] = a[e];
+          qv.v[e + 4] = b[e];
+        }
+        s = mma_wide_a(qv, Frag<T>::load(cs + (kt * 16 + col) * LDC + c + g * 8), s);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) ss[half][g * 4 + i][kt * 16 + col] = s[i];
+    }
+    __syncthreads();
+    {
+      float v[2], p[2];
+      float mt = -INFINITY;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const int key = k0 + sk + 16 * j;
+        const bool see = real && key < hi && key <= pos && pos - key < window;
+        v[j] = see ? (ss[0][srow][sk + 16 * j] + ss[1][srow][sk + 16 * j]) * scale : -INFINITY;
+        mt = fmaxf(mt, v[j]);
+      }
+#pragma unroll
+      for (int o = 8; o > 0; o >>= 1) mt = fmaxf(mt, __shfl_xor(mt, o, 64));
+      const float mn = fmaxf(m, mt);
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        p[j] = mn == -INFINITY ? 0.f : expf(v[j] - mn);
+        sum += p[j];
+        ps[srow][sk + 16 * j] = p[j];
+      }
+#pragma unroll
+      for (int o = 8; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
+      const float a = mn == -INFINITY ? 1.f : expf(m - mn);
+      l = l * a + sum;
+      m = mn;
+      if (sk == 0) al[srow] = a;
+    }
+    __syncthreads();
+    {
+      Wide8 pv;
+      const f32x4_t a = load4(&ps[col][g * 8]), b = load4(&ps[col][g * 8 + 4]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        pv.v[e] = a[e];
+        pv.v[e + 4] = b[e];
+      }
+      f32x4_t f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) f[i] = al[g * 4 + i];
+#pragma unroll
+      for (int i = 0; i < NCT; ++i) {
+        const int c = (wave + 4 * i) * 16 + col;
+        Frag<T> cf;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) cf.set(e, (float)cs[(g * 8 + e) * LDC + c]);
+        acc[i] = mma_wide_a(pv, cf, acc[i] * f);
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < NCT; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (q0 + g * 4 + j < rows) ctx[(slot + q0 + g * 4 + j) * RANK + (wave + 4 * i) * 16 + col] = acc[i][j];
+  if (sk == 0 && real) {
+    ml[(slot + q0 + srow) * 2] = m;
+    ml[(slot + q0 + srow) * 2 + 1] = l;
+  }
+}
+
+// Splits of one (row, head) combined, value projection and output gate.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict__ ctx, const float* __restrict__ ml,
+                                                         const T* __restrict__ uv, const T* __restrict__ gate, long ldg,
+                                                         T* __restrict__ out, long ldo, const int32_t* __restrict__ n_dev,
+                                                         int R, int H, int splits, int dvp, int rank) {
+  extern __shared__ __align__(16) unsigned char smem[];
+  float* cs = reinterpret_cast<float*>(smem);     // [rank]
+  float* ws = cs + rank;                          // [splits]
+  const int r = blockIdx.x, h = blockIdx.y;
+  if (r >= hyb_live(n_dev, R)) return;
+  const size_t row = (size_t)r * H + h, stride = (size_t)R * H;
+  float m = -INFINITY;
+  for (int s = 0; s < splits; ++s) m = fmaxf(m, ml[(s * stride + row) * 2]);
+  float l = 0.f;
+  for (int s = 0; s < splits; ++s) {
+    const float ms = ml[(s * stride + row) * 2];
+    l += ms == -INFINITY ? 0.f : expf(ms - m) * ml[(s * stride + row) * 2 + 1];
+  }
+  for (int s = threadIdx.x; s < splits; s += 256) {
+    const float ms = ml[(s * stride + row) * 2];
+    ws[s] = ms == -INFINITY ? 0.f : expf(ms - m) / l;
+  }
+  __syncthreads();
+  for (int d = threadIdx.x; d < rank; d += 256) {
+    float v = 0.f;
+    for (int s = 0; s < splits; ++s)
+      if (ws[s] != 0.f) v = fmaf(ws[s], ctx[(s * stride + row) * rank + d], v);
+    cs[d] = v;
+  }
+  __syncthreads();
+  // eight lanes per value row
+  const int sub = threadIdx.x & 7;
+  for (int v0 = threadIdx.x >> 3; v0 < dvp; v0 += 32) {
+    const T* w = uv + ((size_t)h * dvp + v0) * rank;
+    float a = 0.f;
+    for (int d = sub * 8; d < rank; d += 64) {
+      const Frag<T> f = Frag<T>::load(w + d);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) a = fmaf(f.at(e), cs[d + e], a);
+    }
+    a += __shfl_xor(a, 1, 64);
+    a += __shfl_xor(a, 2, 64);
+    a += __shfl_xor(a, 4, 64);
+    if (sub == 0) {
+      const size_t c = (size_t)h * dvp + v0;
+      out[(size_t)r * ldo + c] = (T)(a * hyb_sigmoid((float)gate[(size_t)r * ldg + c]));
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------
+// Windowed causal attention of a prompt portion over projected keys and values.
+// k [S][ldk] (head h at h dp), vt [H dvp][ldv] transposed; row s is position base + s with
+// base = max(0, len - back).  Four waves of 16 QT query rows; 64 keys per step.  Scores are formed
+// transposed (keys x queries), so a lane keeps one query per tile: the softmax needs two lane
+// exchanges per step and the weights are the second product's operand as they stand.
+// ------------------------------------------------------------------------------------
+template <typename T>
+__device__ inline Frag<T> frag_halves(const T* a, const T* b) {      // four elements from each
+  Frag<T> f;
+  if constexpr (sizeof(T) == 2) {
+    const bf16x4_t x = *reinterpret_cast<const bf16x4_t*>(a), y = *reinterpret_cast<const bf16x4_t*>(b);
+    f.v = bf16x8_t{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+  } else {
+    f.lo = *reinterpret_cast<const f32x4_t*>(a);
+    f.hi = *reinterpret_cast<const f32x4_t*>(b);
+  }
+  return f;
+}
+
+template <typename T, int C, int QT>
+__global__ __launch_bounds__(256) void window_attention_kernel(
+    const T* __restrict__ q, long ldq, const T* __restrict__ k, long ldk, const T* __restrict__ vt, long ldv,
+    const T* __restrict__ gate, long ldg, T* __restrict__ out, long ldo, const int32_t* __restrict__ len_dev,
+    const int32_t* __restrict__ n_dev, int R, int dp, int dvp, int window, int back, float scale) {
+  constexpr int ND = C / 32, NV = C / 16, KT = 64;
+  constexpr int EPC = 16 / sizeof(T);
+  constexpr int LDK = C + EPC, LDV = KT + EPC;
+  constexpr int KCH = C / EPC, VCH = KT / EPC;               // 16-byte chunks per row
+  constexpr int KI = KT * KCH / 256, VI = C * VCH / 256;     // chunks per thread
+  __shared__ __align__(16) T ks[KT * LDK];
+  __shared__ __align__(16) T vs[C * LDV];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y;
+  const int live = hyb_live(n_dev, R);
+  // the portion's last rows see the most keys where the window does not cut: start with them
+  const int q0 = (gridDim.x - 1 - blockIdx.x) * 64 * QT;
+  if (q0 >= live) return;
+  const int len = *len_dev;
+  const int base = len > back ? len - back : 0;
+  const int qend = q0 + 64 * QT < live ? q0 + 64 * QT : live;
+  int lo = len + q0 - window + 1 - base;
+  lo = lo > 0 ? lo & ~(KT - 1) : 0;
+  const int hi = len + qend - base;                          // keys [lo, hi) as rows of k
+
+  Frag<T> qf[QT][ND];
+  int qpos[QT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int r = q0 + wave * 16 * QT + t * 16 + col;
+    qpos[t] = len + r - base;
+    const T* qr = q + (size_t)(r < live ? r : live - 1) * ldq + (size_t)h * dp + g * 8;
+#pragma unroll
+    for (int s = 0; s < ND; ++s) qf[t][s] = s * 32 < dp ? Frag<T>::load(qr + s * 32) : Frag<T>::zero();
+  }
+  f32x4_t acc[NV][QT];
+#pragma unroll
+  for (int v = 0; v < NV; ++v)
+#pragma unroll
+    for (int t = 0; t < QT; ++t) acc[v][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float m[QT], l[QT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    m[t] = -1e30f;
+    l[t] = 0.f;
+  }
+  const float sc = scale * LOG2E;
+
+  u32x4_t kr[KI], vr[VI];
+  const int kch = dp / EPC;
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < KI; ++i) {
+      const int c = tid + 256 * i, row = c / KCH, ch = c % KCH;
+      if (ch < kch) kr[i] = *reinterpret_cast<const u32x4_t*>(k + (size_t)(k0 + row) * ldk + (size_t)h * dp + ch * EPC);
+    }
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+      const int c = tid + 256 * i, row = c / VCH, ch = c % VCH;
+      if (row < dvp) vr[i] = *reinterpret_cast<const u32x4_t*>(vt + ((size_t)h * dvp + row) * ldv + k0 + ch * EPC);
+    }
+  };
+  auto put = [&]() {
+#pragma unroll
+    for (int i = 0; i < KI; ++i) {
+      const int c = tid + 256 * i, row = c / KCH, ch = c % KCH;
+      if (ch < kch) *reinterpret_cast<u32x4_t*>(ks + row * LDK + ch * EPC) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+      const int c = tid + 256 * i, row = c / VCH, ch = c % VCH;
+      if (row < dvp) *reinterpret_cast<u32x4_t*>(vs + row * LDV + ch * EPC) = vr[i];
+    }
+  };
+  fetch(lo);
+  for (int k0 = lo; k0 < hi; k0 += KT) {
+    put();
+    __syncthreads();
+    if (k0 + KT < hi) fetch(k0 + KT);
+    f32x4_t s[4][QT];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt) {
+#pragma unroll
+      for (int t = 0; t < QT; ++t) s[kt][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int d = 0; d < ND; ++d)
+        if (d * 32 < dp) {
+          const Frag<T> kf = Frag<T>::load(ks + (kt * 16 + col) * LDK + d * 32 + g * 8);
+#pragma unroll
+          for (int t = 0; t < QT; ++t) s[kt][t] = mma(kf, qf[t][d], s[kt][t]);
+        }
+    }
+    const bool edge = k0 + KT > len + q0 - base + 1 || len + qend - base - k0 > window;
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      float mt = -1e30f;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float v = s[kt][t][i] * sc;
+          if (edge) {
+            const int back_by = qpos[t] - (k0 + kt * 16 + g * 4 + i);
+            v = back_by >= 0 && back_by < window ? v : -INFINITY;
+          }
+          s[kt][t][i] = v;
+          mt = fmaxf(mt, v);
+        }
+      mt = fmaxf(mt, __shfl_xor(mt, 16, 64));
+      mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
+      const float mn = fmaxf(m[t], mt), a = __builtin_amdgcn_exp2f(m[t] - mn);
+      float sum = 0.f;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float e = __builtin_amdgcn_exp2f(s[kt][t][i] - mn);
+          s[kt][t][i] = e;
+          sum += e;
+        }
+      l[t] = l[t] * a + sum;
+      m[t] = mn;
+#pragma unroll
+      for (int v = 0; v < NV; ++v) acc[v][t] *= a;
+    }
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      Frag<T> ph[QT], pl[QT];
+#pragma unroll
+      for (int t = 0; t < QT; ++t) {
+        Wide8 w;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          w.v[e] = s[2 * p][t][e];
+          w.v[e + 4] = s[2 * p + 1][t][e];
+        }
+        if constexpr (sizeof(T) == 2)
+          split(w, ph[t], pl[t]);
+        else
+          ph[t] = as_frag(w);
+      }
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+        if (v * 16 < dvp) {
+          const T* vp = vs + (v * 16 + col) * LDV + p * 32 + g * 4;
+          const Frag<T> vf = frag_halves<T>(vp, vp + 16);
+#pragma unroll
+          for (int t = 0; t < QT; ++t) {
+            if constexpr (sizeof(T) == 2) acc[v][t] = mma(vf, pl[t], acc[v][t]);
+            acc[v][t] = mma(vf, ph[t], acc[v][t]);
+          }
+        }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    float lt = l[t];
+    lt += __shfl_xor(lt, 16, 64);
+    lt += __shfl_xor(lt, 32, 64);
+    const int r = q0 + wave * 16 * QT + t * 16 + col;
+    if (r >= live) continue;
+    const float inv = 1.f / lt;
+#pragma unroll
+    for (int v = 0; v < NV; ++v)
+      if (v * 16 < dvp) {
+        const size_t c = (size_t)h * dvp + v * 16 + g * 4;
+        const f32x4_t gt = load4(gate + (size_t)r * ldg + c);
+        f32x4_t o = acc[v][t] * inv;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] *= hyb_sigmoid(gt[i]);
+        store4<T>(out + (size_t)r * ldo + c, o);
+      }
+  }
+}
+
+// keys per split and number of splits of the absorbed form: about 128 workgroups per launch
+void split_plan(int R, int H, int window, long cap, int* keys, int* splits) {
+  long span = (long)window - 1 + R;
+  if (span > cap) span = cap;
+  const long groups = ((long)R * H + 15) / 16;
+  long per = span * groups / 128;
+  per = (per + 31) / 32 * 32;
+  if (per < 64) per = 64;
+  long n = (span + per - 1) / per;
+  if (n > 1024) {
+    per = ((span + 1023) / 1024 + 31) / 32 * 32;
+    n = (span + per - 1) / per;
+  }
+  *keys = (int)per;
+  *splits = (int)n;
+}
+
+template <typename T, int NCT>
+void launch_split(const float* qa, const void* cache, const int32_t* len, const int32_t* n, float* ctx, float* ml, int R,
+                  int H, int window, float scale, int keys, int splits, long cap, hipStream_t st) {
+  constexpr int RANK = NCT * 64;
+  const size_t lds = 32 * (RANK * sizeof(T) + 16);
+  static bool big = false;
+  if (!big && lds > 65536) {      // dynamic LDS beyond 64 KB has to be asked for
+    (void)hipFuncSetAttribute((const void*)latent_split_kernel<T, NCT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    big = true;
+  }
+  latent_split_kernel<T, NCT><<<dim3((R * H + 15) / 16, splits), 256, lds, st>>>(qa, (const T*)cache, len, n, ctx, ml, R, H,
+                                                                                window, scale, keys, cap);
+}
+template <typename T>
+int dispatch_split(int nct, const float* qa, const void* cache, const int32_t* len, const int32_t* n, float* ctx, float* ml,
+                   int R, int H, int window, float scale, int keys, int splits, long cap, hipStream_t st) {
+  switch (nct) {
+#define CASE(X) \
+  case X: launch_split<T, X>(qa, cache, len, n, ctx, ml, R, H, window, scale, keys, splits, cap, st); return HYB_OK;
+    CASE(1) CASE(2) CASE(3) CASE(4) CASE(5) CASE(6) CASE(7) CASE(8) CASE(12) CASE(16)
+#undef CASE
+  }
+  return HYB_ERR_SHAPE;
+}
+template <typename T, int C, int QT>
+void launch_window(const hyb_window_args* a, hipStream_t st) {
+  const dim3 grid((a->R + 64 * QT - 1) / (64 * QT), a->H);
+  window_attention_kernel<T, C, QT><<<grid, 256, 0, st>>>((const T*)a->q, a->ldq, (const T*)a->k, a->ldk, (const T*)a->vt,
+                                                          a->ldv, (const T*)a->gate, a->ldg, (T*)a->out, a->ldo, a->len_dev,
+                                                          a->n_dev, a->R, a->dp, a->dvp, a->window, a->back, a->scale);
+}
+
+}  // namespace
+
+HYB_EXPORT int hyb_latent_append(int dtype, const void* x, long ldx, const float* w, float eps, void* cache, long cap,
+                                 const int32_t* len_dev, const int32_t* n_dev, int R, int rank, int rank_true,
+                                 hyb_stream_t stream) {
+  if (!x || !w || !cache || !len_dev) return HYB_ERR_NULL;
+  if (dtype != HYB_BF16 && dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (R < 1 || rank < 64 || rank % 64 || rank_true < 1 || rank_true > rank || cap < 1 || ldx < rank || ldx % 8)
+    return HYB_ERR_SHAPE;
+  if (!hyb_aligned16(x) || !hyb_aligned16(w) || !hyb_aligned16(cache)) return HYB_ERR_ALIGN;
+  HYB_DISPATCH(dtype, latent_append_kernel<T><<<(R + 3) / 4, 256, 0, (hipStream_t)stream>>>(
+                          (const T*)x, ldx, w, eps, (T*)cache, cap, len_dev, n_dev, R, rank, rank_true);)
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_latent_rank_supported(int rank) {
+  if (rank < 64 || rank % 64) return 0;
+  const int n = rank / 64;
+  return n <= 8 || n == 12 || n == 16;
+}
+
+HYB_EXPORT size_t hyb_latent_decode_workspace_bytes(int R, int H, int rank, int window, long cap) {
+  if (R < 1 || H < 1 || !hyb_latent_rank_supported(rank) || window < 1 || cap < 1) return 0;
+  int keys, splits;
+  split_plan(R, H, window, cap, &keys, &splits);
+  const size_t rows = (size_t)R * H;
+  return (rows * rank + (size_t)splits * rows * (rank + 2)) * 4;
+}
+
+HYB_EXPORT int hyb_latent_decode(const hyb_latent_decode_args* a, hyb_stream_t stream) {
+  if (!a || !a->q || !a->cache || !a->uk || !a->uv || !a->gate || !a->out || !a->len_dev) return HYB_ERR_NULL;
+  if (a->dtype != HYB_BF16 && a->dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (a->R < 1 || a->R > 64 || a->H < 1 || a->dp < 1 || a->dvp < 1 || !hyb_latent_rank_supported(a->rank) || a->window < 1 ||
+      a->cap < 1)
+    return HYB_ERR_SHAPE;
+  if (a->ldq < (long)a->H * a->dp || a->ldg < (long)a->H * a->dvp || a->ldo < (long)a->H * a->dvp) return HYB_ERR_SHAPE;
+  if (!hyb_aligned16(a->cache) || !hyb_aligned16(a->uk) || !hyb_aligned16(a->uv)) return HYB_ERR_ALIGN;
+  if (!a->workspace || a->workspace_bytes < hyb_latent_decode_workspace_bytes(a->R, a->H, a->rank, a->window, a->cap))
+    return HYB_ERR_WORKSPACE;
+  int keys, splits;
+  split_plan(a->R, a->H, a->window, a->cap, &keys, &splits);
+  const size_t rows = (size_t)a->R * a->H;
+  float* qa = (float*)a->workspace;
+  float* ctx = qa + rows * a->rank;
+  float* ml = ctx + (size_t)splits * rows * a->rank;
+  hipStream_t st = (hipStream_t)stream;
+  int rc = HYB_OK;
+  HYB_DISPATCH(
+      a->dtype,
+      absorb_kernel<T><<<dim3(a->H, a->rank / 64), 256, 0, st>>>((const T*)a->q, a->ldq, (const T*)a->uk, qa, a->n_dev, a->R,
+                                                                 a->H, a->dp, a->rank);
+      rc = dispatch_split<T>(a->rank / 64, qa, a->cache, a->len_dev, a->n_dev, ctx, ml, a->R, a->H, a->window, a->scale, keys,
+                             splits, a->cap, st);
+      latent_out_kernel<T><<<dim3(a->R, a->H), 256, (size_t)(a->rank + splits) * 4, st>>>(
+          ctx, ml, (const T*)a->uv, (const T*)a->gate, a->ldg, (T*)a->out, a->ldo, a->n_dev, a->R, a->H, splits, a->dvp,
+          a->rank);)
+  if (rc != HYB_OK) return rc;
+  return hyb_launch_status();
+}
+
+HYB_EXPORT int hyb_window_attention(const hyb_window_args* a, hyb_stream_t stream) {
+  if (!a || !a->q || !a->k || !a->vt || !a->gate || !a->out || !a->len_dev) return HYB_ERR_NULL;
+  if (a->dtype != HYB_BF16 && a->dtype != HYB_F32) return HYB_ERR_UNSUPPORTED;
+  if (a->R < 1 || a->H < 1 || a->dp < 32 || a->dp % 32 || a->dp > 256 || a->dvp < 16 || a->dvp % 16 || a->dvp > 256 ||
+      a->window < 1 || a->back < 0 || a->back > a->window - 1)
+    return HYB_ERR_SHAPE;
+  // keys are read in whole steps of 64 rows
+  if (a->ldq < (long)a->H * a->dp || a->ldk < (long)a->H * a->dp || a->ldg < (long)a->H * a->dvp ||
+      a->ldo < (long)a->H * a->dvp || a->ldq % 8 || a->ldk % 8 || a->ldg % 4 || a->ldo % 4 || a->ldv % 64 ||
+      a->ldv < (long)a->back + a->R)
+    return HYB_ERR_SHAPE;
+  if (!hyb_aligned16(a->q) || !hyb_aligned16(a->k) || !hyb_aligned16(a->vt) || !hyb_aligned16(a->gate) || !hyb_aligned16(a->out))
+    return HYB_ERR_ALIGN;
+  const int c = a->dp > a->dvp ? a->dp : a->dvp;
+  const bool many = (long)((a->R + 127) / 128) * a->H >= 192;
+  hipStream_t st = (hipStream_t)stream;
+  HYB_DISPATCH(
+      a->dtype,
+      if (c <= 64) { many ? launch_window<T, 64, 2>(a, st) : launch_window<T, 64, 1>(a, st); } else if (c <= 128) {
+        many ? launch_window<T, 128, 2>(a, st) : launch_window<T, 128, 1>(a, st);
+      } else launch_window<T, 256, 1>(a, st);)
+  return hyb_launch_status();
+}

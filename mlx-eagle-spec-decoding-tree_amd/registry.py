@@ -1,0 +1,55 @@
+"""Model families the framework serves: how a checkpoint's config.json selects one, which storage types
+it runs in, which library its kernels are in, and how it is loaded."""
+from dataclasses import dataclass
+from typing import Callable, Tuple
+
+
+@dataclass(frozen=True)
+class Family:
+    name: str
+    matches: Callable[[dict], bool]
+    load: Callable            # (path, config, device, dtype name or None) -> model
+    libraries: Tuple[str, ...]
+    dtypes: Tuple[str, ...]   # first: what it is served in
+
+
+_FAMILIES = []
+
+
+def register(family):
+    _FAMILIES.append(family)
+    return family
+
+
+def resolve(config):
+    """The family of a config.json.  Without an 'architecture' entry it is the quantised Llama / Qwen2
+    decoder, whose reader checks the rest."""
+    for f in _FAMILIES:
+        if f.matches(config):
+            return f
+    raise ValueError(f"no model family serves architecture {config.get('architecture')!r}")
+
+
+def names():
+    return [f.name for f in _FAMILIES]
+
+
+def _load_lositar(path, config, device, dtype):
+    import torch
+
+    from . import lositar
+    return lositar.load(path, config, device, getattr(torch, dtype) if dtype else None)
+
+
+def _load_llama(path, config, device, dtype):
+    from . import checkpoint, llama
+    if dtype not in (None, "float16"):
+        raise ValueError(f"the quantised decoder computes in float16, not {dtype}")
+    args = checkpoint.model_args_from_config(config)
+    weights = checkpoint.load_weights(path, device)
+    checkpoint.check_quantized(args, weights)
+    return llama.Model(args, weights, device)
+
+
+register(Family("lositar", lambda c: c.get("architecture") == "Lositar", _load_lositar, ("hybrid",), ("bfloat16", "float32")))
+register(Family("llama", lambda c: "architecture" not in c, _load_llama, ("eagle",), ("float16",)))
