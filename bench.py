@@ -186,6 +186,10 @@ def main():
                          "1 GiB read + 1 GiB written) so that profiler byte counters can be scaled")
     ap.add_argument("--loop", action="store_true",
                     help="measure the end-to-end tree loop (drafter + target) instead of the verify step")
+    ap.add_argument("--hybrid", action="store_true",
+                    help="prefill and decode throughput of a Lositar decoder (linear + latent attention, bf16) beside "
+                         "the quantised Llama decoder of equal size, with every kernel's share of its roofline")
+    ap.add_argument("--hybrid-sizes", default="small,large", help="--hybrid: which of small, large to run")
     ap.add_argument("--gemm", action="store_true",
                     help="measure the many-row (prompt pass) form of the quantised matmul instead")
     ap.add_argument("--small-m", action="store_true",
@@ -217,6 +221,9 @@ def main():
         if opt.steps == 50:
             opt.steps = 300
         print(json.dumps(loop_bench(opt)), flush=True)
+        return
+    if opt.hybrid:
+        print(json.dumps(hybrid_bench(opt)), flush=True)
         return
     if opt.gemm:
         print(json.dumps(gemm_bench(opt)), flush=True)
@@ -499,6 +506,226 @@ def main():
     if parity is not None and not parity["ok"]:
         print("bench.py: full-size parity check failed (see `parity` in the line above)", file=sys.stderr)
         sys.exit(1)
+
+
+class LaunchRecorder:
+    """Records the calls that a pass makes to functions of an operator module, so that the launches of
+    one kind can be timed on their own: every layer's in turn, as one HIP graph."""
+
+    def __init__(self, module, names):
+        self.module, self.names, self.calls = module, names, []
+
+    def __enter__(self):
+        self.saved = {n: getattr(self.module, n) for n in self.names}
+        for n, fn in self.saved.items():
+            def record(*a, _n=n, _fn=fn, **k):
+                self.calls.append((_n, _fn, a, k))
+                return _fn(*a, **k)
+            setattr(self.module, n, record)
+        return self
+
+    def __exit__(self, *exc):
+        for n, fn in self.saved.items():
+            setattr(self.module, n, fn)
+
+    def table(self, torch, kind):
+        """kind(name, args, kwargs) -> (label, bytes, flops, flop peak in TFLOP/s); {label: row}."""
+        groups = {}
+        for name, fn, a, k in self.calls:
+            label, nbytes, flops, peak = kind(name, a, k)
+            g = groups.setdefault(label, [[], nbytes, flops, peak])
+            g[0].append((fn, a, k))
+        rows = {}
+        for label, (calls, nbytes, flops, peak) in groups.items():
+            # at least eight launches per replay, so that starting the graph does not count
+            reps = -(-8 // len(calls))
+            def run():
+                for _ in range(reps):
+                    for fn, a, k in calls:
+                        fn(*a, **k)
+            ms, _ = graph_time_ms(torch, run, reps=9)
+            us = 1e3 * sorted(ms)[len(ms) // 2] / (reps * len(calls))
+            gbs, tf = nbytes / us / 1e3, flops / us / 1e6
+            by_flops = bool(peak) and flops / (peak * 1e6) > nbytes / (HBM_PEAK_GBS * 1e3)
+            rows[label] = {"calls": len(calls), "us": round(us, 2), "gbs": round(gbs, 1), "tflops": round(tf, 2),
+                           "bound": "flops" if by_flops else "hbm",
+                           "frac": round(tf / peak if by_flops else gbs / HBM_PEAK_GBS, 4)}
+        return rows
+
+
+BF16_PEAK, F32_MATRIX_PEAK = 2500.0, 157.3      # dense TFLOP/s
+
+
+def lositar_cost(prompt, context, window):
+    """kind() of LaunchRecorder.table for a pass of `prompt` rows after `context` cached tokens."""
+    def kind(name, a, k):
+        if name == "dense":
+            x, w, out = a[:3]
+            M = k.get("M") or x.shape[0]
+            N, K = w.shape
+            if k.get("len_dev") is not None:
+                M = min(M, min(context, k["back"]) + prompt)
+            folded = ", norm folded in" if k.get("norm") else ""
+            return (f"dense {M} x {N} x {K}{folded}", 2.0 * N * K + 2.0 * M * K + out.element_size() * M * N,
+                    2.0 * M * N * K, BF16_PEAK)
+        if name in ("gla_step", "gla_chunks"):
+            H, dk, dv = (a[5] if name == "gla_step" else a[4]).shape
+            io = 2.0 * prompt * H * (2 * dk + 3 * dv)
+            if name == "gla_step":
+                return "linear attention, recurrence", 8.0 * H * dk * dv + io, 4.0 * prompt * H * dk * dv, F32_MATRIX_PEAK
+            c = 64
+            return ("linear attention, chunks", io + 4.0 * prompt * H * dk,
+                    prompt * H * (4.0 * dk * dv + (c + 1.0) * (dk + dv)), F32_MATRIX_PEAK)
+        if name == "latent_decode":
+            uk, uv, H, dp, dvp = a[2], a[3], a[9], a[10], a[11]
+            keys = min(window, context + 1)
+            rank = uk.shape[1]
+            return ("latent attention, absorbed", 2.0 * rank * (keys + H * (dp + dvp)),
+                    prompt * H * (4.0 * keys * rank + 2.0 * rank * (dp + dvp)), BF16_PEAK)
+        if name == "window_attention":
+            H, dp, dvp = a[8], a[9], a[10]
+            keys = sum(min(window, context + i + 1) for i in range(prompt))
+            return ("window attention", 2.0 * H * (prompt + min(context, window)) * (dp + dvp) + 4.0 * prompt * H * dvp,
+                    2.0 * H * keys * (dp + dvp), BF16_PEAK)
+        if name == "norm_rows":
+            out = a[4]
+            return "norm", 6.0 * out.shape[0] * out.shape[1], 0.0, 0.0
+        if name == "embed":
+            return "embedding", 8.0 * a[7].shape[0] * a[7].shape[1], 0.0, 0.0
+        if name == "latent_append":
+            return "latent norm + append", 4.0 * prompt * a[4].shape[1], 0.0, 0.0
+        return name, 4.0 * a[0].numel(), 0.0, 0.0
+    return kind
+
+
+def llama_cost(prompt, context):
+    def kind(name, a, k):
+        if name in ("quantized_matmul", "quantized_matmul_swiglu", "quantized_matmul_slabs", "quantized_matmul_small"):
+            x, w = a[0], a[1]
+            M, K, N = x.shape[0], x.shape[-1], w.shape[0]
+            folded = ", norm folded in" if k.get("norm_weight") is not None else ""
+            return f"{name} {M} x {N} x {K}{folded}", qmm_bytes(M, N, K), 2.0 * M * N * K, BF16_PEAK
+        if name in ("causal_attention", "draft_attention"):
+            H, _, hd = a[0].shape
+            G = a[1].shape[0]
+            keys = sum(context + i + 1 for i in range(prompt))
+            return name, 4.0 * G * (context + prompt) * hd + 4.0 * H * prompt * hd, 4.0 * H * keys * hd, BF16_PEAK
+        if name in ("rms_norm", "rms_norm_slabs"):
+            D = a[1].shape[-1] if name == "rms_norm" else a[2].shape[-1]
+            return name, (8.0 if k.get("residual") is not None else 4.0) * prompt * D, 0.0, 0.0
+        if name == "embed":
+            return name, 2.6 * prompt * a[1].shape[1] * 8, 0.0, 0.0
+        t = a[0]
+        return name, 2.0 * t.numel() * t.element_size(), 0.0, 0.0
+    return kind
+
+
+def hybrid_bench(opt):
+    """Prompt pass of 2048 tokens and greedy decoding behind it, random weights, eight layers that
+    resemble a 1B / 8B model's: the Lositar decoder in bf16 beside the quantised Llama decoder with the
+    same width, heads and (to 2 %) weights per layer."""
+    import torch
+    from mlx_eagle_spec_decoding_tree_amd import (_lib, generate, hybrid, hybrid_ops, llama, lositar, ops, spec,
+                                                  synth)
+
+    dev = torch.device("cuda:0")
+    _lib.check(_lib.lib().eagle_check_device(), "device check")
+    P, V, layers, window = 2048, 65536, 8, 1024
+    steps = max(opt.steps, 50)
+    sizes = {"small": dict(width=2048, heads=16, ff=8192, inter=5504), "large": dict(width=4096, heads=32, ff=16384, inter=11008)}
+    out = {}
+
+    def times(fn, reps=9):
+        ms, _ = graph_time_ms(torch, fn, reps=reps)
+        return sorted(ms)[len(ms) // 2]
+
+    for name in opt.hybrid_sizes.split(","):
+        z = sizes[name]
+        res = {"width": z["width"], "layers": layers, "heads": z["heads"], "head_dim": 128, "prompt": P, "window": window}
+        # ---- Lositar ----
+        cfg = synth.lositar_config(width=z["width"], layers=layers, heads=z["heads"], ff=z["ff"], vocab=V, window=window,
+                                   max_positions=2 * P + 64)
+        model = lositar.build(cfg, synth.make_lositar_weights(cfg, opt.seed, dev), dev)
+        stream = generate.open_stream(model, 2 * P)
+        ids = torch.randint(0, V, (P,), generator=torch.Generator().manual_seed(opt.seed))
+        logits = stream.feed(ids)
+        first = stream.pick(logits)
+        stream.greedy(first, 4)
+        big = stream.passes[P]
+        live = torch.tensor([P], dtype=torch.int32, device=dev)
+        start = torch.zeros(1, dtype=torch.int32, device=dev)
+
+        def prefill():
+            big.len_dev.copy_(start)
+            big.n_dev.copy_(live)
+            big.enqueue()
+        ms_p = times(prefill)
+        dec = stream._decode
+        one = torch.ones(1, dtype=torch.int32, device=dev)
+        ctx = torch.tensor([P], dtype=torch.int32, device=dev)
+
+        def decode():
+            dec.p.n_dev.copy_(one)
+            dec.p.len_dev.copy_(ctx)
+            dec.enqueue()
+        ms_d = times(decode, reps=steps)
+        names = ["dense", "gla_step", "gla_chunks", "latent_decode", "window_attention", "norm_rows", "embed", "latent_append"]
+        with LaunchRecorder(hybrid_ops, names) as rec:
+            prefill()
+        tab_p = rec.table(torch, lositar_cost(P, 0, window))
+        with LaunchRecorder(hybrid_ops, names) as rec:
+            decode()
+        big.len_dev.copy_(ctx)
+        tab_d = rec.table(torch, lositar_cost(1, P, window))
+        n_w = sum(t.numel() for layer in model.layers for t in (layer.mixer.proj, layer.mixer.o, layer.mlp.up, layer.mlp.down))
+        res["lositar"] = {"dtype": "bf16", "weights_per_layer": round(n_w / layers), "prefill_ms": round(ms_p, 3),
+                          "prefill_tokens_per_s": round(P / ms_p * 1e3), "decode_ms": round(ms_d, 4),
+                          "decode_tokens_per_s": round(1e3 / ms_d, 1), "prefill_kernels": tab_p, "decode_kernels": tab_d}
+        print(f"[bench] {name} lositar: prefill {ms_p:.3f} ms, decode {ms_d:.4f} ms", file=sys.stderr, flush=True)
+        del model, stream, big, dec, rec
+        # ---- Llama ----
+        la = synth.ModelArgs(model_type="llama", hidden_size=z["width"], num_hidden_layers=layers, intermediate_size=z["inter"],
+                             num_attention_heads=z["heads"], num_key_value_heads=z["heads"], head_dim=128, vocab_size=V,
+                             rope_theta=5e5, tie_word_embeddings=True)
+        model = llama.Model.from_numpy(la, synth.make_model_weights(la, seed=opt.seed), dev)
+        stream = generate.open_stream(model, 2 * P)
+        logits = stream.feed(ids)
+        first = stream.pick(logits)
+        stream.greedy(first, 4)
+        big = stream._prefill.passes[P]
+
+        def prefill():
+            big.len_dev.copy_(start)
+            big.enqueue()
+        ms_p = times(prefill)
+
+        def decode():
+            stream.cache[0].len_dev.copy_(ctx)
+            stream._step()
+        ms_d = times(decode, reps=steps)
+        names = ["quantized_matmul", "quantized_matmul_swiglu", "quantized_matmul_slabs", "quantized_matmul_small",
+                 "causal_attention", "draft_attention", "rms_norm", "rms_norm_slabs", "rope_kv_append", "qkv_rope_small", "embed"]
+        with LaunchRecorder(ops, names) as rec:
+            prefill()
+        tab_p = rec.table(torch, llama_cost(P, 0))
+        with LaunchRecorder(ops, names) as rec:
+            decode()
+        big.len_dev.copy_(ctx)
+        tab_d = rec.table(torch, llama_cost(1, P))
+        at, mlp = model.layers[0].self_attn, model.layers[0].mlp
+        n_w = 8 * sum(l.weight.numel() for l in (at.q_proj, at.k_proj, at.v_proj, at.o_proj, mlp.gate_proj, mlp.up_proj, mlp.down_proj))
+        res["llama"] = {"dtype": "4-bit weights, f16", "weights_per_layer": n_w, "prefill_ms": round(ms_p, 3),
+                        "prefill_tokens_per_s": round(P / ms_p * 1e3), "decode_ms": round(ms_d, 4),
+                        "decode_tokens_per_s": round(1e3 / ms_d, 1), "prefill_kernels": tab_p, "decode_kernels": tab_d}
+        print(f"[bench] {name} llama: prefill {ms_p:.3f} ms, decode {ms_d:.4f} ms", file=sys.stderr, flush=True)
+        del model, stream, big, rec
+        out[name] = res
+    last = out[list(out)[-1]]
+    return {"metric": "Lositar decoder, prompt tokens per second", "value": last["lositar"]["prefill_tokens_per_s"], "unit": "tokens/s",
+            "n_gpus": 1, "steps": steps, "warmup": opt.warmup, "ms_per_step": last["lositar"]["prefill_ms"], "higher_is_better": True,
+            "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "8 layers, 2048-token prompt pass, greedy decode behind it, beside the quantised Llama decoder"},
+            "sizes": out}
 
 
 def gemm_bench(opt):

@@ -60,7 +60,7 @@ class LlamaStream:
         self._check(n)
         if (want is None or list(want) == [n - 1]) and n > 1:
             if self._prefill is None:
-                self._prefill = spec.CausalPrefill(self.model, self.cache, graphs=False)
+                self._prefill = spec.CausalPrefill(self.model, self.cache, chunk=spec.MAX_CHUNK, graphs=False)
             return self._prefill(ids).float()
         rows = [n - 1] if want is None else [int(w) for w in want]
         logits = self.model(ids[None], cache=self.cache)[0]
@@ -72,31 +72,52 @@ class LlamaStream:
         from . import ops
         return int(ops.argmax_rows(logits[-1:].half()).item())
 
-    def greedy(self, token, n):
-        from . import _lib, ops, spec
+    def _step(self):
+        from . import _lib, ops
 
+        L, st, length = _lib.lib(), torch.cuda.current_stream().cuda_stream, self.cache[0].len_dev
+        _lib.check(L.eagle_tree_positions(self._zero.data_ptr(), length.data_ptr(), self._pos.data_ptr(), 1, st), "positions")
+        logits = self._pass.forward(self._y, self._pos, length, length, self._mask, 1)
+        ops.argmax_rows(logits, out=self._y)
+        _lib.check(L.eagle_advance_len(length.data_ptr(), 1, st), "advance_len")
+
+    def _prepare_step(self):
+        from . import ops, spec
+
+        i32 = dict(dtype=torch.int32, device=self.model.device)
+        self._pass = spec.DecoderPass(self.model, self.cache, 1)
+        self._y, self._zero, self._pos = torch.zeros(1, **i32), torch.zeros(1, **i32), torch.zeros(1, **i32)
+        self._mask = ops.mask_to_words(torch.ones((1, 1), dtype=torch.bool, device=self.model.device))
+        self._out = torch.zeros(self.MAX_OUT, **i32)
+        if not self.graphs:
+            return
+        # the warm-up run writes one cache row beyond the length and advances the length
+        length = self.cache[0].len_dev
+        saved = length.clone()
+        side = torch.cuda.Stream()
+        side.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(side):
+            self._step()
+        torch.cuda.current_stream().wait_stream(side)
+        torch.cuda.synchronize()
+        self._graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(self._graph):
+            self._step()
+        length.copy_(saved)
+
+    def greedy(self, token, n):
         self._check(n)
         if n > self.MAX_OUT:
             return (first := self.greedy(token, self.MAX_OUT)) + self.greedy(first[-1], n - self.MAX_OUT)
-        i32 = dict(dtype=torch.int32, device=self.model.device)
-        if self._pass is None:
-            self._pass = spec.DecoderPass(self.model, self.cache, 1)
-            self._y, self._zero, self._pos = torch.zeros(1, **i32), torch.zeros(1, **i32), torch.zeros(1, **i32)
-            self._mask = ops.mask_to_words(torch.ones((1, 1), dtype=torch.bool, device=self.model.device))
-            self._out = torch.zeros(self.MAX_OUT, **i32)
-        p, length, L = self._pass, self.cache[0].len_dev, _lib.lib()
-
-        def step():
-            st = torch.cuda.current_stream().cuda_stream
-            _lib.check(L.eagle_tree_positions(self._zero.data_ptr(), length.data_ptr(), self._pos.data_ptr(), 1, st), "positions")
-            logits = p.forward(self._y, self._pos, length, length, self._mask, 1)
-            ops.argmax_rows(logits, out=self._y)
-            _lib.check(L.eagle_advance_len(length.data_ptr(), 1, st), "advance_len")
-
         self.cache[0].sync_len()
+        if self._pass is None:
+            self._prepare_step()
         self._y.fill_(int(token))
         for i in range(n):
-            step()
+            if self._graph is not None:
+                self._graph.replay()
+            else:
+                self._step()
             self._out[i:i + 1].copy_(self._y)
         self._set_length(self.length + n)
         return self._out[:n].tolist()

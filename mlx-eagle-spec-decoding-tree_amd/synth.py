@@ -164,6 +164,54 @@ def make_model_weights(args: ModelArgs, seed=42, layers=None, gain=1.0):
     return out
 
 
+def lositar_config(width=2048, layers=8, heads=16, dim=128, vdim=128, rank=512, ff=8192, vocab=65536, window=1024,
+                   tau=16.0, max_positions=8192, eps=1e-5, embed_scale=1.0):
+    """config.json of a Lositar model: latent attention on even layers (the second, fourth, ... of them with the
+    latents of the one before), linear attention on odd ones."""
+    out = []
+    for i in range(layers):
+        if i % 2:
+            mixer = {"heads": heads, "dim": dim, "vdim": vdim, "tau": tau}
+        else:
+            mixer = {"heads": heads, "dim": dim, "vdim": vdim, "kv_rank": rank, "scale": dim ** -0.5,
+                     "mask": {"size": window}}
+            if i % 4 == 2:
+                mixer["kv_from"] = i - 2
+        out.append({"type": "gla" if i % 2 else "latent_attention", "mixer": mixer,
+                    "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Lositar", "vocab": vocab, "width": width, "max_positions": max_positions,
+            "norm": {"eps": eps}, "embedding": {"scale": embed_scale}, "layers": out}
+
+
+def make_lositar_weights(config, seed=42, device="cpu", decay_rank=16):
+    """Random bf16 tensors of a Lositar checkpoint as a flat dict of torch tensors."""
+    import torch
+
+    from . import hybrid, lositar
+
+    gen = torch.Generator(device=device).manual_seed(seed)
+    shapes = hybrid.Model.shapes(lositar.args_from_config(config))
+    flat = {k: v for k, v in shapes.items() if k != "layers"}
+    for i, layer in enumerate(shapes["layers"]):
+        flat.update({f"l{i}.{k}": v for k, v in layer.items()})
+    out = {}
+    for name, shape in flat.items():
+        shape = tuple(decay_rank if n is None else n for n in shape)
+        t = torch.randn(shape, generator=gen, device=device)
+        if name.endswith(("norm1", "norm2", "final.norm")):
+            t = 0.1 * t
+        elif name.endswith((".dkv.norm", "mix.norm")):
+            t = 1.0 + 0.1 * t
+        elif name.endswith("a2.b"):
+            t = 1.0 + t
+        elif name == "pos":
+            t = 0.3 * t
+        elif name != "embed":
+            t = t * shape[-1] ** -0.5
+        out[name] = t.to(torch.bfloat16)
+    return out
+
+
 def inv_freqs(args: ModelArgs, seq_len=None):
     """fp32 inverse-frequency table and scaling factor of the rotary embedding
     (mlx_llama.py:98-116).
