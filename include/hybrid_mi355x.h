@@ -114,11 +114,12 @@ int hyb_latent_append(int dtype, const void* x, long ldx, const float* w, float 
                       const int32_t* len_dev, const int32_t* n_dev, int R, int rank, int rank_true, hyb_stream_t stream);
 
 /* Latent attention of few rows (R <= 64) with absorbed key projection: position i = *len_dev + r sees the cached
- * rows j with 0 <= i - j < window (its own row is appended already).  q [R][ldq] (H x dp), uk [H dp][rank],
+ * rows j with 0 <= i - j < window.  append [R][ldappend]: the new rows before their norm, normed and appended
+ * first as by hyb_latent_append; NULL where they are in the cache already.  q [R][ldq] (H x dp), uk [H dp][rank],
  * uv [H dvp][rank], gate [R][ldg] (H x dvp): out[r] = (softmax(scale q.k) v) * sigmoid(gate). */
 typedef struct {
   const void* q;
-  const void* cache;
+  void* cache;
   const void* uk;
   const void* uv;
   const void* gate;
@@ -127,9 +128,11 @@ typedef struct {
   const int32_t* n_dev;
   void* workspace;
   size_t workspace_bytes;
-  long ldq, ldg, ldo, cap;
-  int dtype, R, H, dp, dvp, rank, window;
-  float scale;
+  const void* append;
+  const float* append_norm;
+  long ldq, ldg, ldo, cap, ldappend;
+  int dtype, R, H, dp, dvp, rank, window, rank_true;
+  float scale, eps;
 } hyb_latent_decode_args;
 int hyb_latent_rank_supported(int rank);
 size_t hyb_latent_decode_workspace_bytes(int R, int H, int rank, int window, long cap);

@@ -118,8 +118,9 @@ HybGlaArgs = _struct("HybGlaArgs", (c_void_p, "x a2 a2_bias z norm_w state out n
                      (c_size_t, "workspace_bytes"), (c_long, "ldx ldo"),
                      (c_int, "dtype R H dkp dvp rp dv_true off_q off_k off_v off_g off_a"), (c_float, "qscale tau eps"))
 HybLatentDecodeArgs = _struct("HybLatentDecodeArgs", (c_void_p, "q cache uk uv gate out len_dev n_dev workspace"),
-                              (c_size_t, "workspace_bytes"), (c_long, "ldq ldg ldo cap"),
-                              (c_int, "dtype R H dp dvp rank window"), (c_float, "scale"))
+                              (c_size_t, "workspace_bytes"), (c_void_p, "append append_norm"),
+                              (c_long, "ldq ldg ldo cap ldappend"),
+                              (c_int, "dtype R H dp dvp rank window rank_true"), (c_float, "scale eps"))
 HybWindowArgs = _struct("HybWindowArgs", (c_void_p, "q k vt gate out len_dev n_dev"), (c_long, "ldq ldk ldv ldg ldo"),
                         (c_int, "dtype R H dp dvp window back"), (c_float, "scale"))
 

@@ -261,7 +261,7 @@ __global__ __launch_bounds__(512) void dense_skinny_kernel(DenseP p) {
 // (double buffered, 16-byte chunks xored with the row so that reads spread over the banks).
 // TRANS: the block is stored transposed, out[n][m].
 template <typename T, int BM, int BN, bool TRANS>
-__global__ __launch_bounds__(256) void dense_gemm_kernel(DenseP p, int tiles_m, int tiles_n) {
+__global__ __launch_bounds__(256, 2) void dense_gemm_kernel(DenseP p, int tiles_m, int tiles_n) {
   constexpr int BK = 128 / sizeof(T), EPC = 16 / sizeof(T);
   constexpr int TM = BM / 32, TN = BN / 32, SUB = BK / 32;
   __shared__ __align__(16) unsigned char lds[2][(BM + BN) * 128];
@@ -403,9 +403,10 @@ void launch_gemm(const DenseP& p, hipStream_t st) {
 template <typename T>
 void dense_gemm(const DenseP& p, hipStream_t st) {
   auto blocks = [&](int bm, int bn) { return (long)((p.M + bm - 1) / bm) * ((p.N + bn - 1) / bn); };
-  if (blocks(128, 128) >= 256)
+  // two workgroups for every compute unit, or one over a K long enough to pay for the larger block
+  if (blocks(128, 128) >= 512 || (blocks(128, 128) >= 256 && p.K >= 4096))
     launch_gemm<T, 128, 128>(p, st);
-  else if (blocks(64, 128) >= 256)
+  else if (blocks(64, 128) >= 512)
     launch_gemm<T, 64, 128>(p, st);
   else
     launch_gemm<T, 64, 64>(p, st);

@@ -218,24 +218,51 @@ __global__ __launch_bounds__(256, 2) void gla_chunk_kernel(ChunkP p) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) A[(I * SUBC + g * 4 + i) * CH + J * SUBC + col] = acc[i];
   }
-  // diagonal tile of this wave: lane = (j, quarter of d), one row i after the other
+  // Diagonal tile of this wave: lane = (j, quarter of d), one row i after the other.  128 columns at a time
+  // with this lane's keys and decays in registers; the next row's queries are requested ahead.
   {
+    constexpr int DB = 4;
     const int b0 = wave * SUBC, rj = b0 + col;
-#pragma unroll 1
-    for (int i = 0; i < SUBC; ++i) {
-      float s = 0.f;
-      for (int d = g * 8; d < dkp; d += 32) {
-        const Frag<T> k = row8<T>(p, r0 + rj, live, p.ok + h * dkp + d);
-        const Frag<T> q = row8<T>(p, r0 + b0 + i, live, p.oq + h * dkp + d);
-        const Frag<float> lj = Frag<float>::load(Ls + rj * ldl + d), li = Frag<float>::load(Ls + (b0 + i) * ldl + d);
+    for (int d0 = 0; d0 < dkp; d0 += 32 * DB) {
+      Frag<T> k[DB], q[DB];
+      Frag<float> lj[DB];
+      int at[DB];
 #pragma unroll
-        for (int e = 0; e < 8; ++e)       // j > i is dropped below: only keep the exponent in range
-          s = fmaf(q.at(e) * k.at(e), decay_exp(fminf(li.at(e) - lj.at(e), 0.f)), s);
+      for (int t = 0; t < DB; ++t) {
+        const int d = d0 + t * 32 + g * 8;
+        at[t] = d < dkp ? d : dkp - 8;
+        k[t] = d < dkp ? row8<T>(p, r0 + rj, live, p.ok + h * dkp + d) : Frag<T>::zero();
+        lj[t] = Frag<float>::load(Ls + rj * ldl + at[t]);
       }
-      s *= p.qscale;
-      s += __shfl_xor(s, 16, 64);
-      s += __shfl_xor(s, 32, 64);
-      if (g == 0) A[(b0 + i) * CH + rj] = col <= i ? s : 0.f;
+      auto queries = [&](int i) {
+        const int r = r0 + b0 + i < live ? r0 + b0 + i : live - 1;      // rows past the live ones are not used
+        const T* x = reinterpret_cast<const T*>(p.x) + (size_t)r * p.ldx + p.oq + h * dkp;
+#pragma unroll
+        for (int t = 0; t < DB; ++t) q[t] = Frag<T>::load(x + at[t]);
+      };
+      queries(0);
+#pragma unroll 1
+      for (int i = 0; i < SUBC; ++i) {
+        float s = 0.f;
+        Frag<T> now[DB];
+#pragma unroll
+        for (int t = 0; t < DB; ++t) now[t] = q[t];
+        if (i + 1 < SUBC) queries(i + 1);
+#pragma unroll
+        for (int t = 0; t < DB; ++t) {
+          const Frag<float> li = Frag<float>::load(Ls + (b0 + i) * ldl + at[t]);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)       // j > i is dropped below: only keep the exponent in range
+            s = fmaf(now[t].at(e) * k[t].at(e), decay_exp(fminf(li.at(e) - lj[t].at(e), 0.f)), s);
+        }
+        s *= p.qscale;
+        s += __shfl_xor(s, 16, 64);
+        s += __shfl_xor(s, 32, 64);
+        if (g == 0) {
+          float* o = A + (b0 + i) * CH + rj;
+          *o = (d0 ? *o : 0.f) + (col <= i ? s : 0.f);
+        }
+      }
     }
   }
   __syncthreads();
@@ -255,22 +282,34 @@ __global__ __launch_bounds__(256, 2) void gla_chunk_kernel(ChunkP p) {
     for (int d = tid; d < dkp; d += 256)
       p.decay[((size_t)c * p.H + h) * dkp + d] = decay_exp(Ts[d] + Ts[dkp + d] + Ts[2 * dkp + d] + Ts[3 * dkp + d]);
   __syncthreads();
-  // U = K^T V: each wave takes value tiles, all key tiles
+  // U = K^T V.  Value columns go in groups of 64: tile j of a group holds columns 4 c + j, so that a lane
+  // reads and writes four columns at once.  The waves share a group's key tiles where there are few groups.
   float* U = p.U + ((size_t)c * p.H + h) * dkp * p.dvp;
-  for (int vt = wave; vt < (p.dvp >> 4); vt += 4) {
-    float vv[16];
+  const int groups = (p.dvp + 63) >> 6, share = groups == 1 ? 4 : (groups == 2 ? 2 : 1);
+  for (int vg = wave / share; vg < groups; vg += 4 / share) {
+    const int v0 = vg * 64 + col * 4, vc = v0 < p.dvp ? v0 : p.dvp - 4;
+    f32x4_t vv[16];
 #pragma unroll
     for (int s = 0; s < 16; ++s) {
-      const int r = r0 + 4 * s + g;
-      vv[s] = r < live ? (float)reinterpret_cast<const T*>(p.x)[(size_t)r * p.ldx + p.ov + h * p.dvp + vt * 16 + col] : 0.f;
+      const int r = r0 + 4 * s + g;       // keys past the live rows are zero
+      vv[s] = load4(reinterpret_cast<const T*>(p.x) + (size_t)(r < live ? r : live - 1) * p.ldx + p.ov + h * p.dvp + vc);
     }
-    for (int dt = 0; dt < (dkp >> 4); ++dt) {
-      f32x4_t acc = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int dt = wave % share; dt < (dkp >> 4); dt += share) {
+      f32x4_t acc[4];
 #pragma unroll
-      for (int s = 0; s < 16; ++s)
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(Ls[(4 * s + g) * ldl + dt * 16 + col], vv[s], acc, 0, 0, 0);
+      for (int j = 0; j < 4; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < 4; ++i) U[(size_t)(dt * 16 + g * 4 + i) * p.dvp + vt * 16 + col] = acc[i];
+      for (int s = 0; s < 16; ++s) {
+        const float k = Ls[(4 * s + g) * ldl + dt * 16 + col];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, vv[s][j], acc[j], 0, 0, 0);
+      }
+      if (v0 < p.dvp) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          *reinterpret_cast<f32x4_t*>(U + (size_t)(dt * 16 + g * 4 + i) * p.dvp + v0) =
+              f32x4_t{acc[0][i], acc[1][i], acc[2][i], acc[3][i]};
+      }
     }
   }
 }
@@ -304,7 +343,8 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(ChunkP p) {
   *reinterpret_cast<f32x4_t*>(p.state + at) = s;
 }
 
-template <typename T, int NVT>
+// NG: groups of 64 value columns (tile j of a group: columns 4 c + j)
+template <typename T, int NG>
 __global__ __launch_bounds__(256) void gla_out_kernel(ChunkP p) {
   extern __shared__ __align__(16) float sm[];
   const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -330,22 +370,32 @@ __global__ __launch_bounds__(256) void gla_out_kernel(ChunkP p) {
   __syncthreads();
   const float* S = p.U + ((size_t)c * p.H + h) * dkp * dvp;
   const float* A = p.A + ((size_t)c * p.H + h) * CH * CH + (wave * SUBC + col) * CH + g * 8;
-  const int nvt = dvp >> 4;
-  f32x4_t acc[NVT];
+  const T* V = reinterpret_cast<const T*>(p.x) + p.ov + h * dvp;
+  int vc[NG];                              // this lane's columns (groups past the last repeat it)
 #pragma unroll
-  for (int v = 0; v < NVT; ++v) acc[v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int v = 0; v < NG; ++v) vc[v] = v * 64 + col * 4 < dvp ? v * 64 + col * 4 : dvp - 4;
+  f32x4_t acc[NG][4];
+#pragma unroll
+  for (int v = 0; v < NG; ++v)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[v][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  auto add = [&](const Frag<float>& a, const f32x4_t (&b)[8], f32x4_t (&o)[4]) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) o[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a.at(e), b[e][j], o[j], 0, 0, 0);
+  };
   for (int d = g * 8; d < (dkp + 31) / 32 * 32; d += 32) {
     const bool in = d < dkp;
     const Frag<float> q = in ? Frag<float>::load(Qs + (wave * SUBC + col) * ldq + d) : Frag<float>::zero();
-    const float* Sr = S + (size_t)(in ? d : 0) * dvp + col;
+    const float* Sr = S + (size_t)(in ? d : 0) * dvp;
 #pragma unroll
-    for (int v = 0; v < NVT; ++v)
-      if (v < nvt) {
-        Frag<float> b;
+    for (int v = 0; v < NG; ++v) {
+      f32x4_t b[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) b.set(e, Sr[e * dvp + v * 16]);
-        acc[v] = mma(q, b, acc[v]);
-      }
+      for (int e = 0; e < 8; ++e) b[e] = load4(Sr + e * dvp + vc[v]);
+      add(q, b, acc[v]);
+    }
   }
   // within the chunk: rows of A against V (32 rows at a time, no further than this wave's rows)
   for (int j0 = 0; j0 < (wave < 2 ? 32 : 64); j0 += 32) {
@@ -354,23 +404,24 @@ __global__ __launch_bounds__(256) void gla_out_kernel(ChunkP p) {
     // tiles above the diagonal are never written
     if ((jr >> 4) > wave) a = Frag<float>::zero();
 #pragma unroll
-    for (int v = 0; v < NVT; ++v)
-      if (v < nvt) {
-        Frag<float> b;
+    for (int v = 0; v < NG; ++v) {
+      f32x4_t b[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const int r = r0 + jr + e;
-          b.set(e, r < live ? (float)reinterpret_cast<const T*>(p.x)[(size_t)r * p.ldx + p.ov + h * dvp + v * 16 + col] : 0.f);
-        }
-        acc[v] = mma(a, b, acc[v]);
+      for (int e = 0; e < 8; ++e) {
+        const int r = r0 + jr + e < live ? r0 + jr + e : live - 1;      // a's columns past the live rows are zero
+        b[e] = load4(V + (size_t)r * p.ldx + vc[v]);
       }
+      add(a, b, acc[v]);
+    }
   }
   float ss[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int v = 0; v < NVT; ++v)
-    if (v < nvt) {
+  for (int v = 0; v < NG; ++v)
+    if (v * 64 + col * 4 < dvp) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) ss[i] += acc[v][i] * acc[v][i];
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) ss[i] += acc[v][j][i] * acc[v][j][i];
     }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
@@ -379,16 +430,19 @@ __global__ __launch_bounds__(256) void gla_out_kernel(ChunkP p) {
     ss[i] = 1.f / sqrtf(ss[i] / (float)p.dv_true + p.eps);
   }
 #pragma unroll
-  for (int v = 0; v < NVT; ++v)
-    if (v < nvt) {
-      const float w = p.norm_w[v * 16 + col];
+  for (int v = 0; v < NG; ++v)
+    if (v * 64 + col * 4 < dvp) {
+      const f32x4_t w = load4(p.norm_w + vc[v]);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int r = r0 + wave * SUBC + g * 4 + i;
         if (r < live) {
-          const int at = h * dvp + v * 16 + col;
-          const float gt = (float)reinterpret_cast<const T*>(p.x)[(size_t)r * p.ldx + p.og + at];
-          reinterpret_cast<T*>(p.out)[(size_t)r * p.ldo + at] = (T)(acc[v][i] * ss[i] * w * gt * hyb_sigmoid(gt));
+          const int at = h * dvp + vc[v];
+          const f32x4_t gt = load4(reinterpret_cast<const T*>(p.x) + (size_t)r * p.ldx + p.og + at);
+          f32x4_t o;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) o[j] = acc[v][j][i] * ss[i] * w[j] * gt[j] * hyb_sigmoid(gt[j]);
+          store4<T>(reinterpret_cast<T*>(p.out) + (size_t)r * p.ldo + at, o);
         }
       }
     }
@@ -428,17 +482,15 @@ void launch_chunks(const ChunkP& p, hipStream_t st) {
 #define OUT(N)                             \
   allow_lds(gla_out_kernel<T, N>, lds3);   \
   gla_out_kernel<T, N><<<grid, 256, lds3, st>>>(p)
-  const int nvt = p.dvp / 16;
-  if (nvt <= 2) {
+  const int ng = (p.dvp + 63) / 64;
+  if (ng == 1) {
+    OUT(1);
+  } else if (ng == 2) {
     OUT(2);
-  } else if (nvt <= 4) {
+  } else if (ng <= 4) {
     OUT(4);
-  } else if (nvt <= 8) {
-    OUT(8);
-  } else if (nvt <= 16) {
-    OUT(16);
   } else {
-    OUT(32);
+    OUT(8);
   }
 #undef OUT
 }
@@ -450,7 +502,9 @@ int check_gla(const hyb_gla_args* a) {
       a->dv_true < 1 || a->dv_true > a->dvp || a->tau <= 0.f || a->ldx % 8 || a->ldo < (long)a->H * a->dvp)
     return HYB_ERR_SHAPE;
   if (a->off_q % 8 || a->off_k % 8 || a->off_v % 8 || a->off_g % 8 || a->off_a % 8) return HYB_ERR_ALIGN;
-  if (!hyb_aligned16(a->x) || !hyb_aligned16(a->state) || !hyb_aligned16(a->a2)) return HYB_ERR_ALIGN;
+  if (!hyb_aligned16(a->x) || !hyb_aligned16(a->state) || !hyb_aligned16(a->a2) || !hyb_aligned16(a->norm_w) ||
+      !hyb_aligned16(a->out) || a->ldo % 8)
+    return HYB_ERR_ALIGN;
   return HYB_OK;
 }
 

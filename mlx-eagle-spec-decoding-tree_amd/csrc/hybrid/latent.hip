@@ -16,50 +16,66 @@ constexpr float LOG2E = 1.4426950408889634f;
 // ------------------------------------------------------------------------------------
 // c = norm(W_dkv h) into cache row len + r.  One wave per row.
 // ------------------------------------------------------------------------------------
+struct AppendP {
+  const void* x;           // NULL: nothing to append
+  const float* w;
+  void* cache;
+  long ldx, cap;
+  int rank, rank_true;
+  float eps;
+};
 template <typename T>
-__global__ __launch_bounds__(256) void latent_append_kernel(const T* __restrict__ x, long ldx,
-                                                            const float* __restrict__ w, float eps, T* __restrict__ cache,
-                                                            long cap, const int32_t* __restrict__ len_dev,
-                                                            const int32_t* __restrict__ n_dev, int R, int rank, int rank_true) {
-  const int r = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (r >= hyb_live(n_dev, R)) return;
-  const long row = (long)*len_dev + r;
-  if (row >= cap) return;                       // the host checks the capacity; never write past it
-  const T* xr = x + (size_t)r * ldx;
+__device__ inline void append_row(const AppendP& p, int r, long row, int lane) {
+  if (row >= p.cap) return;                     // the host checks the capacity; never write past it
+  const T* xr = reinterpret_cast<const T*>(p.x) + (size_t)r * p.ldx;
   float ss = 0.f;
-  for (int d = lane * 4; d < rank; d += 256) {
+  for (int d = lane * 4; d < p.rank; d += 256) {
     const f32x4_t v = load4(xr + d);
     ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
   }
   ss = hyb_wave_sum(ss);
-  const float rstd = 1.f / sqrtf(ss / (float)rank_true + eps);
-  for (int d = lane * 4; d < rank; d += 256) store4<T>(cache + (size_t)row * rank + d, load4(xr + d) * rstd * load4(w + d));
+  const float rstd = 1.f / sqrtf(ss / (float)p.rank_true + p.eps);
+  T* out = reinterpret_cast<T*>(p.cache) + (size_t)row * p.rank;
+  for (int d = lane * 4; d < p.rank; d += 256) store4<T>(out + d, load4(xr + d) * rstd * load4(p.w + d));
+}
+template <typename T>
+__global__ __launch_bounds__(256) void latent_append_kernel(AppendP p, const int32_t* __restrict__ len_dev,
+                                                            const int32_t* __restrict__ n_dev, int R) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (r < hyb_live(n_dev, R)) append_row<T>(p, r, (long)*len_dev + r, threadIdx.x & 63);
 }
 
 // ------------------------------------------------------------------------------------
 // Absorbed queries, fp32: qa[r][h][:] = sum_d q[r][h][d] W_uk[h dp + d][:].
-// Workgroup = one head and 64 latent columns; 32 groups of eight lanes share d.
+// Workgroup = one head and 64 latent columns; 32 groups of eight lanes share d; MR rows at a time.
+// The last plane of the grid appends the new rows to the cache.
 // ------------------------------------------------------------------------------------
-template <typename T>
+template <typename T, int MR>
 __global__ __launch_bounds__(256) void absorb_kernel(const T* __restrict__ q, long ldq, const T* __restrict__ uk,
-                                                     float* __restrict__ qa, const int32_t* __restrict__ n_dev, int R, int H,
-                                                     int dp, int rank) {
-  __shared__ float red[4][4][64];
-  const int h = blockIdx.x, c0 = blockIdx.y * 64;
+                                                     float* __restrict__ qa, const int32_t* __restrict__ len_dev,
+                                                     const int32_t* __restrict__ n_dev, int R, int H, int dp, int rank,
+                                                     AppendP ap) {
+  __shared__ float red[4][MR][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int cl = (lane & 7) * 8, dg = wave * 8 + (lane >> 3);
   const int live = hyb_live(n_dev, R);
+  if ((int)blockIdx.y == rank / 64) {
+    const long len = *len_dev;
+    for (int r = blockIdx.x * 4 + wave; r < live; r += gridDim.x * 4) append_row<T>(ap, r, len + r, lane);
+    return;
+  }
+  const int h = blockIdx.x, c0 = blockIdx.y * 64;
+  const int cl = (lane & 7) * 8, dg = wave * 8 + (lane >> 3);
   const T* wk = uk + (size_t)h * dp * rank + c0 + cl;
-  for (int r0 = 0; r0 < live; r0 += 4) {
-    float acc[4][8];
+  for (int r0 = 0; r0 < live; r0 += MR) {
+    float acc[MR][8];
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
+    for (int r = 0; r < MR; ++r)
 #pragma unroll
       for (int e = 0; e < 8; ++e) acc[r][e] = 0.f;
     for (int d = dg; d < dp; d += 32) {
       const Frag<T> w = Frag<T>::load(wk + (size_t)d * rank);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
+      for (int r = 0; r < MR; ++r) {
         const int rr = r0 + r < live ? r0 + r : live - 1;
         const float qv = (float)q[(size_t)rr * ldq + h * dp + d];
 #pragma unroll
@@ -67,7 +83,7 @@ __global__ __launch_bounds__(256) void absorb_kernel(const T* __restrict__ q, lo
       }
     }
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
+    for (int r = 0; r < MR; ++r)
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         float v = acc[r][e];
@@ -78,7 +94,8 @@ __global__ __launch_bounds__(256) void absorb_kernel(const T* __restrict__ q, lo
       }
     __syncthreads();
     const int r = threadIdx.x >> 6, c = threadIdx.x & 63;
-    if (r0 + r < live) qa[((size_t)(r0 + r) * H + h) * rank + c0 + c] = red[0][r][c] + red[1][r][c] + red[2][r][c] + red[3][r][c];
+    if (r < MR && r0 + r < live)
+      qa[((size_t)(r0 + r) * H + h) * rank + c0 + c] = red[0][r][c] + red[1][r][c] + red[2][r][c] + red[3][r][c];
     __syncthreads();
   }
 }
@@ -132,6 +149,24 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const float* __restri
 #pragma unroll
   for (int i = 0; i < NCT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
+  // this wave's part of the queries: 16 keys and every second step of 32 columns per wave
+  constexpr bool HELD = NCT <= 8;
+  const int kt = wave & 1, half = wave >> 1;
+  auto query = [&](int st) {
+    Wide8 v;
+    const f32x4_t a = load4(qrow + (2 * st + half) * 32), b = load4(qrow + (2 * st + half) * 32 + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v.v[e] = a[e];
+      v.v[e + 4] = b[e];
+    }
+    return v;
+  };
+  Wide8 held[HELD ? NCT : 1];
+  if (HELD) {
+#pragma unroll
+    for (int st = 0; st < NCT; ++st) held[HELD ? st : 0] = query(st);
+  }
 
   for (int k0 = lo; k0 < hi; k0 += 32) {
     // stage 32 cached vectors (rows past the end repeat the last one; their weight is zero)
@@ -142,20 +177,11 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const float* __restri
     }
     __syncthreads();
     {
-      const int kt = wave & 1, half = wave >> 1;             // 16 keys, every second step of 32 columns
       f32x4_t s = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int st = 0; st < NCT; ++st) {
-        const int c = (2 * st + half) * 32;
-        Wide8 qv;
-        const f32x4_t a = load4(qrow + c), b = load4(qrow + c + 4);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          qv.v[e] = a[e];
-          qv.v[e + 4] = b[e];
-        }
-        s = mma_wide_a(qv, Frag<T>::load(cs + (kt * 16 + col) * LDC + c + g * 8), s);
-      }
+      for (int st = 0; st < NCT; ++st)
+        s = mma_wide_a(HELD ? held[HELD ? st : 0] : query(st),
+                       Frag<T>::load(cs + (kt * 16 + col) * LDC + (2 * st + half) * 32 + g * 8), s);
 #pragma unroll
       for (int i = 0; i < 4; ++i) ss[half][g * 4 + i][kt * 16 + col] = s[i];
     }
@@ -221,54 +247,83 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const float* __restri
   }
 }
 
-// Splits of one (row, head) combined, value projection and output gate.
-template <typename T>
+// Splits of one (row, head) combined, value projection (32 value rows per workgroup, eight lanes each;
+// their weights are requested first) and output gate.
+template <typename T, int NCT>
 __global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict__ ctx, const float* __restrict__ ml,
                                                          const T* __restrict__ uv, const T* __restrict__ gate, long ldg,
                                                          T* __restrict__ out, long ldo, const int32_t* __restrict__ n_dev,
-                                                         int R, int H, int splits, int dvp, int rank) {
+                                                         int R, int H, int splits, int dvp) {
+  constexpr int RANK = NCT * 64, COLS = RANK / 4, GROUPS = 256 / COLS;
   extern __shared__ __align__(16) unsigned char smem[];
-  float* cs = reinterpret_cast<float*>(smem);     // [rank]
-  float* ws = cs + rank;                          // [splits]
-  const int r = blockIdx.x, h = blockIdx.y;
+  float* ws = reinterpret_cast<float*>(smem);     // [splits]
+  __shared__ __align__(16) float part[GROUPS][RANK];
+  __shared__ float red[8];
+  const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   if (r >= hyb_live(n_dev, R)) return;
-  const size_t row = (size_t)r * H + h, stride = (size_t)R * H;
-  float m = -INFINITY;
-  for (int s = 0; s < splits; ++s) m = fmaxf(m, ml[(s * stride + row) * 2]);
-  float l = 0.f;
-  for (int s = 0; s < splits; ++s) {
-    const float ms = ml[(s * stride + row) * 2];
-    l += ms == -INFINITY ? 0.f : expf(ms - m) * ml[(s * stride + row) * 2 + 1];
-  }
-  for (int s = threadIdx.x; s < splits; s += 256) {
-    const float ms = ml[(s * stride + row) * 2];
-    ws[s] = ms == -INFINITY ? 0.f : expf(ms - m) / l;
-  }
-  __syncthreads();
-  for (int d = threadIdx.x; d < rank; d += 256) {
-    float v = 0.f;
-    for (int s = 0; s < splits; ++s)
-      if (ws[s] != 0.f) v = fmaf(ws[s], ctx[(s * stride + row) * rank + d], v);
-    cs[d] = v;
-  }
-  __syncthreads();
-  // eight lanes per value row
-  const int sub = threadIdx.x & 7;
-  for (int v0 = threadIdx.x >> 3; v0 < dvp; v0 += 32) {
-    const T* w = uv + ((size_t)h * dvp + v0) * rank;
-    float a = 0.f;
-    for (int d = sub * 8; d < rank; d += 64) {
-      const Frag<T> f = Frag<T>::load(w + d);
+  const int sub = tid & 7, v0 = blockIdx.z * 32 + (tid >> 3);
+  Frag<T> w[NCT];
+  {
+    const T* wr = uv + ((size_t)h * dvp + (v0 < dvp ? v0 : dvp - 1)) * RANK + sub * 8;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) a = fmaf(f.at(e), cs[d + e], a);
+    for (int i = 0; i < NCT; ++i) w[i] = Frag<T>::load(wr + i * 64);
+  }
+  const size_t row = (size_t)r * H + h, stride = (size_t)R * H;
+  // weights of the splits: exp(m_s - m) / sum
+  float m = -INFINITY;
+  for (int s = tid; s < splits; s += 256) m = fmaxf(m, ml[(s * stride + row) * 2]);
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
+  if ((tid & 63) == 0) red[tid >> 6] = m;
+  __syncthreads();
+  m = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+  float l = 0.f;
+  for (int s = tid; s < splits; s += 256) {
+    const float ms = ml[(s * stride + row) * 2];
+    const float e = ms == -INFINITY ? 0.f : expf(ms - m);
+    ws[s] = e;
+    l += e * ml[(s * stride + row) * 2 + 1];
+  }
+  l = hyb_wave_sum(l);
+  if ((tid & 63) == 0) red[4 + (tid >> 6)] = l;
+  __syncthreads();
+  const float inv = 1.f / (red[4] + red[5] + red[6] + red[7]);
+  const int cg = tid / COLS, cc = (tid % COLS) * 4;
+  if (cg < GROUPS) {
+    f32x4_t v = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const float* c = ctx + row * RANK + cc;
+#pragma unroll 8
+    for (int s = cg; s < splits; s += GROUPS) {
+      // a split without visible keys has written nothing
+      const f32x4_t x = load4(c + (size_t)s * stride * RANK);
+      const float e = ws[s];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = e != 0.f ? fmaf(e, x[i], v[i]) : v[i];
     }
-    a += __shfl_xor(a, 1, 64);
-    a += __shfl_xor(a, 2, 64);
-    a += __shfl_xor(a, 4, 64);
-    if (sub == 0) {
-      const size_t c = (size_t)h * dvp + v0;
-      out[(size_t)r * ldo + c] = (T)(a * hyb_sigmoid((float)gate[(size_t)r * ldg + c]));
+    *reinterpret_cast<f32x4_t*>(&part[cg][cc]) = v * inv;
+  }
+  __syncthreads();
+  float a = 0.f;
+#pragma unroll
+  for (int i = 0; i < NCT; ++i) {
+    f32x4_t lo = f32x4_t{0.f, 0.f, 0.f, 0.f}, hi = lo;
+#pragma unroll
+    for (int k = 0; k < GROUPS; ++k) {
+      lo += load4(&part[k][i * 64 + sub * 8]);
+      hi += load4(&part[k][i * 64 + sub * 8 + 4]);
     }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      a = fmaf(w[i].at(e), lo[e], a);
+      a = fmaf(w[i].at(e + 4), hi[e], a);
+    }
+  }
+  a += __shfl_xor(a, 1, 64);
+  a += __shfl_xor(a, 2, 64);
+  a += __shfl_xor(a, 4, 64);
+  if (sub == 0 && v0 < dvp) {
+    const size_t c = (size_t)h * dvp + v0;
+    out[(size_t)r * ldo + c] = (T)(a * hyb_sigmoid((float)gate[(size_t)r * ldg + c]));
   }
 }
 
@@ -293,7 +348,7 @@ __device__ inline Frag<T> frag_halves(const T* a, const T* b) {      // four ele
 }
 
 template <typename T, int C, int QT>
-__global__ __launch_bounds__(256) void window_attention_kernel(
+__global__ __launch_bounds__(256, (sizeof(T) == 2 && C <= 128) ? 2 : 1) void window_attention_kernel(
     const T* __restrict__ q, long ldq, const T* __restrict__ k, long ldk, const T* __restrict__ vt, long ldv,
     const T* __restrict__ gate, long ldg, T* __restrict__ out, long ldo, const int32_t* __restrict__ len_dev,
     const int32_t* __restrict__ n_dev, int R, int dp, int dvp, int window, int back, float scale) {
@@ -346,12 +401,12 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
 #pragma unroll
     for (int i = 0; i < KI; ++i) {
       const int c = tid + 256 * i, row = c / KCH, ch = c % KCH;
-      if (ch < kch) kr[i] = *reinterpret_cast<const u32x4_t*>(k + (size_t)(k0 + row) * ldk + (size_t)h * dp + ch * EPC);
+      kr[i] = *reinterpret_cast<const u32x4_t*>(k + (size_t)(k0 + row) * ldk + (size_t)h * dp + (ch < kch ? ch : 0) * EPC);
     }
 #pragma unroll
     for (int i = 0; i < VI; ++i) {
       const int c = tid + 256 * i, row = c / VCH, ch = c % VCH;
-      if (row < dvp) vr[i] = *reinterpret_cast<const u32x4_t*>(vt + ((size_t)h * dvp + row) * ldv + k0 + ch * EPC);
+      vr[i] = *reinterpret_cast<const u32x4_t*>(vt + ((size_t)h * dvp + (row < dvp ? row : 0)) * ldv + k0 + ch * EPC);
     }
   };
   auto put = [&]() {
@@ -367,6 +422,12 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
     }
   };
   fetch(lo);
+  // head sizes below C: the rest of the tiles stays zero, and the products run over it without branches
+  if (dp < C)
+    for (int i = tid; i < KT * LDK; i += 256) ks[i] = (T)0.f;
+  if (dvp < C)
+    for (int i = tid; i < C * LDV; i += 256) vs[i] = (T)0.f;
+  if (dp < C || dvp < C) __syncthreads();
   for (int k0 = lo; k0 < hi; k0 += KT) {
     put();
     __syncthreads();
@@ -377,12 +438,11 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
 #pragma unroll
       for (int t = 0; t < QT; ++t) s[kt][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int d = 0; d < ND; ++d)
-        if (d * 32 < dp) {
-          const Frag<T> kf = Frag<T>::load(ks + (kt * 16 + col) * LDK + d * 32 + g * 8);
+      for (int d = 0; d < ND; ++d) {
+        const Frag<T> kf = Frag<T>::load(ks + (kt * 16 + col) * LDK + d * 32 + g * 8);
 #pragma unroll
-          for (int t = 0; t < QT; ++t) s[kt][t] = mma(kf, qf[t][d], s[kt][t]);
-        }
+        for (int t = 0; t < QT; ++t) s[kt][t] = mma(kf, qf[t][d], s[kt][t]);
+      }
     }
     const bool edge = k0 + KT > len + q0 - base + 1 || len + qend - base - k0 > window;
 #pragma unroll
@@ -434,16 +494,15 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
           ph[t] = as_frag(w);
       }
 #pragma unroll
-      for (int v = 0; v < NV; ++v)
-        if (v * 16 < dvp) {
-          const T* vp = vs + (v * 16 + col) * LDV + p * 32 + g * 4;
-          const Frag<T> vf = frag_halves<T>(vp, vp + 16);
+      for (int v = 0; v < NV; ++v) {
+        const T* vp = vs + (v * 16 + col) * LDV + p * 32 + g * 4;
+        const Frag<T> vf = frag_halves<T>(vp, vp + 16);
 #pragma unroll
-          for (int t = 0; t < QT; ++t) {
-            if constexpr (sizeof(T) == 2) acc[v][t] = mma(vf, pl[t], acc[v][t]);
-            acc[v][t] = mma(vf, ph[t], acc[v][t]);
-          }
+        for (int t = 0; t < QT; ++t) {
+          if constexpr (sizeof(T) == 2) acc[v][t] = mma(vf, pl[t], acc[v][t]);
+          acc[v][t] = mma(vf, ph[t], acc[v][t]);
         }
+      }
     }
     __syncthreads();
   }
@@ -468,42 +527,44 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
   }
 }
 
-// keys per split and number of splits of the absorbed form: about 128 workgroups per launch
+// Keys per split and number of splits of the absorbed form: as little as 32 keys (one tile) per
+// workgroup, at most 64 splits (each is read back by the combining kernel).
 void split_plan(int R, int H, int window, long cap, int* keys, int* splits) {
   long span = (long)window - 1 + R;
   if (span > cap) span = cap;
   const long groups = ((long)R * H + 15) / 16;
-  long per = span * groups / 128;
-  per = (per + 31) / 32 * 32;
-  if (per < 64) per = 64;
-  long n = (span + per - 1) / per;
-  if (n > 1024) {
-    per = ((span + 1023) / 1024 + 31) / 32 * 32;
-    n = (span + per - 1) / per;
-  }
+  long want = 512 / groups;
+  want = want < 1 ? 1 : (want > 64 ? 64 : want);
+  const long per = ((span + want - 1) / want + 31) / 32 * 32;
   *keys = (int)per;
-  *splits = (int)n;
+  *splits = (int)((span + per - 1) / per);
 }
 
 template <typename T, int NCT>
-void launch_split(const float* qa, const void* cache, const int32_t* len, const int32_t* n, float* ctx, float* ml, int R,
-                  int H, int window, float scale, int keys, int splits, long cap, hipStream_t st) {
+void launch_decode(const hyb_latent_decode_args* a, const AppendP& ap, float* qa, float* ctx, float* ml, int keys, int splits,
+                   hipStream_t st) {
   constexpr int RANK = NCT * 64;
+  const dim3 ag(a->H, NCT + (ap.x ? 1 : 0));
+  if (a->R == 1)
+    absorb_kernel<T, 1><<<ag, 256, 0, st>>>((const T*)a->q, a->ldq, (const T*)a->uk, qa, a->len_dev, a->n_dev, a->R, a->H, a->dp,
+                                            RANK, ap);
+  else
+    absorb_kernel<T, 4><<<ag, 256, 0, st>>>((const T*)a->q, a->ldq, (const T*)a->uk, qa, a->len_dev, a->n_dev, a->R, a->H, a->dp,
+                                            RANK, ap);
   const size_t lds = 32 * (RANK * sizeof(T) + 16);
-  static bool big = false;
-  if (!big && lds > 65536) {      // dynamic LDS beyond 64 KB has to be asked for
+  if (lds > 65536)      // dynamic LDS beyond 64 KB has to be asked for
     (void)hipFuncSetAttribute((const void*)latent_split_kernel<T, NCT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    big = true;
-  }
-  latent_split_kernel<T, NCT><<<dim3((R * H + 15) / 16, splits), 256, lds, st>>>(qa, (const T*)cache, len, n, ctx, ml, R, H,
-                                                                                window, scale, keys, cap);
+  latent_split_kernel<T, NCT><<<dim3((a->R * a->H + 15) / 16, splits), 256, lds, st>>>(
+      qa, (const T*)a->cache, a->len_dev, a->n_dev, ctx, ml, a->R, a->H, a->window, a->scale, keys, a->cap);
+  latent_out_kernel<T, NCT><<<dim3(a->R, a->H, (a->dvp + 31) / 32), 256, (size_t)splits * 4, st>>>(
+      ctx, ml, (const T*)a->uv, (const T*)a->gate, a->ldg, (T*)a->out, a->ldo, a->n_dev, a->R, a->H, splits, a->dvp);
 }
 template <typename T>
-int dispatch_split(int nct, const float* qa, const void* cache, const int32_t* len, const int32_t* n, float* ctx, float* ml,
-                   int R, int H, int window, float scale, int keys, int splits, long cap, hipStream_t st) {
-  switch (nct) {
+int dispatch_decode(const hyb_latent_decode_args* a, const AppendP& ap, float* qa, float* ctx, float* ml, int keys, int splits,
+                    hipStream_t st) {
+  switch (a->rank / 64) {
 #define CASE(X) \
-  case X: launch_split<T, X>(qa, cache, len, n, ctx, ml, R, H, window, scale, keys, splits, cap, st); return HYB_OK;
+  case X: launch_decode<T, X>(a, ap, qa, ctx, ml, keys, splits, st); return HYB_OK;
     CASE(1) CASE(2) CASE(3) CASE(4) CASE(5) CASE(6) CASE(7) CASE(8) CASE(12) CASE(16)
 #undef CASE
   }
@@ -527,8 +588,8 @@ HYB_EXPORT int hyb_latent_append(int dtype, const void* x, long ldx, const float
   if (R < 1 || rank < 64 || rank % 64 || rank_true < 1 || rank_true > rank || cap < 1 || ldx < rank || ldx % 8)
     return HYB_ERR_SHAPE;
   if (!hyb_aligned16(x) || !hyb_aligned16(w) || !hyb_aligned16(cache)) return HYB_ERR_ALIGN;
-  HYB_DISPATCH(dtype, latent_append_kernel<T><<<(R + 3) / 4, 256, 0, (hipStream_t)stream>>>(
-                          (const T*)x, ldx, w, eps, (T*)cache, cap, len_dev, n_dev, R, rank, rank_true);)
+  const AppendP p{x, w, cache, ldx, cap, rank, rank_true, eps};
+  HYB_DISPATCH(dtype, latent_append_kernel<T><<<(R + 3) / 4, 256, 0, (hipStream_t)stream>>>(p, len_dev, n_dev, R);)
   return hyb_launch_status();
 }
 
@@ -553,6 +614,9 @@ HYB_EXPORT int hyb_latent_decode(const hyb_latent_decode_args* a, hyb_stream_t s
       a->cap < 1)
     return HYB_ERR_SHAPE;
   if (a->ldq < (long)a->H * a->dp || a->ldg < (long)a->H * a->dvp || a->ldo < (long)a->H * a->dvp) return HYB_ERR_SHAPE;
+  if (a->append && (!a->append_norm || a->ldappend < a->rank || a->ldappend % 8 || a->rank_true < 1 || a->rank_true > a->rank))
+    return a->append_norm ? HYB_ERR_SHAPE : HYB_ERR_NULL;
+  if (!hyb_aligned16(a->append) || !hyb_aligned16(a->append_norm)) return HYB_ERR_ALIGN;
   if (!hyb_aligned16(a->cache) || !hyb_aligned16(a->uk) || !hyb_aligned16(a->uv)) return HYB_ERR_ALIGN;
   if (!a->workspace || a->workspace_bytes < hyb_latent_decode_workspace_bytes(a->R, a->H, a->rank, a->window, a->cap))
     return HYB_ERR_WORKSPACE;
@@ -563,16 +627,9 @@ HYB_EXPORT int hyb_latent_decode(const hyb_latent_decode_args* a, hyb_stream_t s
   float* ctx = qa + rows * a->rank;
   float* ml = ctx + (size_t)splits * rows * a->rank;
   hipStream_t st = (hipStream_t)stream;
+  const AppendP ap{a->append, a->append_norm, a->cache, a->ldappend, a->cap, a->rank, a->rank_true, a->eps};
   int rc = HYB_OK;
-  HYB_DISPATCH(
-      a->dtype,
-      absorb_kernel<T><<<dim3(a->H, a->rank / 64), 256, 0, st>>>((const T*)a->q, a->ldq, (const T*)a->uk, qa, a->n_dev, a->R,
-                                                                 a->H, a->dp, a->rank);
-      rc = dispatch_split<T>(a->rank / 64, qa, a->cache, a->len_dev, a->n_dev, ctx, ml, a->R, a->H, a->window, a->scale, keys,
-                             splits, a->cap, st);
-      latent_out_kernel<T><<<dim3(a->R, a->H), 256, (size_t)(a->rank + splits) * 4, st>>>(
-          ctx, ml, (const T*)a->uv, (const T*)a->gate, a->ldg, (T*)a->out, a->ldo, a->n_dev, a->R, a->H, splits, a->dvp,
-          a->rank);)
+  HYB_DISPATCH(a->dtype, rc = dispatch_decode<T>(a, ap, qa, ctx, ml, keys, splits, st);)
   if (rc != HYB_OK) return rc;
   return hyb_launch_status();
 }
@@ -595,7 +652,7 @@ HYB_EXPORT int hyb_window_attention(const hyb_window_args* a, hyb_stream_t strea
   hipStream_t st = (hipStream_t)stream;
   HYB_DISPATCH(
       a->dtype,
-      if (c <= 64) { many ? launch_window<T, 64, 2>(a, st) : launch_window<T, 64, 1>(a, st); } else if (c <= 128) {
+      if (c <= 32) { many ? launch_window<T, 32, 2>(a, st) : launch_window<T, 32, 1>(a, st); } else if (c <= 64) { many ? launch_window<T, 64, 2>(a, st) : launch_window<T, 64, 1>(a, st); } else if (c <= 128) {
         many ? launch_window<T, 128, 2>(a, st) : launch_window<T, 128, 1>(a, st);
       } else launch_window<T, 256, 1>(a, st);)
   return hyb_launch_status();

@@ -162,18 +162,26 @@ def latent_decode_workspace_bytes(R, H, rank, window, cap):
     return _lib.hybrid().hyb_latent_decode_workspace_bytes(R, H, rank, window, cap)
 
 
-def latent_decode(q, cache, uk, uv, gate, out, len_dev, n_dev, R, H, dp, dvp, window, scale, ws):
-    """Windowed attention of few rows over cached latents (absorbed key projection), gated."""
+def latent_decode(q, cache, uk, uv, gate, out, len_dev, n_dev, R, H, dp, dvp, window, scale, ws,
+                  append=None):
+    """Windowed attention of few rows over cached latents (absorbed key projection), gated.
+    append = (rows [., rank], norm weight, eps, columns that count): the new rows, normed and appended
+    first (None: they are in the cache)."""
     _need_cuda(q, cache, uk, uv, gate, out, ws)
     cap, rank = cache.shape
+    new, new_norm, eps, rank_true = append if append is not None else (None, None, 0.0, 0)
+    if new is not None and (new.shape[0] < R or new.shape[1] < rank or new.dtype != cache.dtype or new_norm.numel() != rank
+                            or new_norm.dtype != torch.float32):
+        raise ValueError("latent_decode: rows to append do not fit")
     if tuple(uk.shape) != (H * dp, rank) or tuple(uv.shape) != (H * dvp, rank) \
             or min(q.shape[0], gate.shape[0], out.shape[0]) < R or q.shape[1] < H * dp or gate.shape[1] < H * dvp \
             or out.shape[1] < H * dvp or len({t.dtype for t in (q, cache, uk, uv, gate, out)}) != 1 \
             or not (cache.is_contiguous() and uk.is_contiguous() and uv.is_contiguous()):
         raise ValueError("latent_decode: shape or type mismatch")
     a = _lib.HybLatentDecodeArgs(_ptr(q), _ptr(cache), _ptr(uk), _ptr(uv), _ptr(gate), _ptr(out), _ptr(len_dev), _ptr(n_dev),
-                                 _ptr(ws), ws.numel(), _rows(q, "q"), _rows(gate, "gate"), _rows(out, "out"), cap,
-                                 code(q.dtype), R, H, dp, dvp, rank, int(window), float(scale))
+                                 _ptr(ws), ws.numel(), _ptr(new), _ptr(new_norm), _rows(q, "q"), _rows(gate, "gate"),
+                                 _rows(out, "out"), cap, 0 if new is None else _rows(new, "append"), code(q.dtype), R, H, dp,
+                                 dvp, rank, int(window), int(rank_true), float(scale), float(eps))
     _lib.check_hybrid(_lib.hybrid().hyb_latent_decode(ctypes.byref(a), _stream()), "latent_decode")
     return out
 

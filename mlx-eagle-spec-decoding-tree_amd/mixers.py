@@ -188,15 +188,16 @@ class LatentAttention(Module):
         p.project(self.proj, norm, x)
         og, oc = H * self.dp, H * (self.dp + self.dvp)
         q, gate = x[:, :og], x[:, og:oc]
-        if s.kv_from is None:
-            hops.latent_append(x[:, oc:], self.dkv_norm, self.eps, s.rank, cache.latents, p.len_dev, p.n_dev, R)
+        new = (x[:, oc:], self.dkv_norm, self.eps, s.rank) if s.kv_from is None else None
         attn = p.buffer("attn", self.o.shape[1])
         window = min(s.window, UNBOUNDED)
         if R <= ABSORB_ROWS:
             ws = p.bytes("latent", hops.latent_decode_workspace_bytes(R, H, self.rank, window, cache.capacity))
             hops.latent_decode(q, cache.latents, self.uk, self.uv, gate, attn, p.len_dev, p.n_dev, R, H, self.dp, self.dvp,
-                               window, s.scale, ws)
+                               window, s.scale, ws, append=new)
         else:
+            if new is not None:
+                hops.latent_append(*new, cache.latents, p.len_dev, p.n_dev, R)
             back = min(window - 1, cache.capacity)
             span = back + R
             S = round_up(span, 128)
