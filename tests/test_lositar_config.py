@@ -1,0 +1,270 @@
+"""Host side of the Lositar family, no GPU: configuration, weight layout, registry, checkpoint, caches,
+the generation command's and the trace runner's logic, and the C ABI's argument checks."""
+import copy
+import ctypes
+import io
+import json
+import os
+import re
+
+import numpy as np
+import pytest
+import torch
+
+from mlx_eagle_spec_decoding_tree_amd import (_lib, cache, checkpoint, generate, hybrid, lositar, mixers, registry, synth,
+                                              trace)
+from lositar_util import CONFIGS, altered, config, gla, latent, weights
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+CPU = torch.device("cpu")
+
+
+def test_args_follow_the_config():
+    a = lositar.args_from_config(CONFIGS["mixed"])
+    assert (a.vocab_size, a.width, a.max_positions, a.norm_eps, a.embed_scale) == (203, 88, 700, 1e-5, 3.0)
+    assert a.num_hidden_layers == 5
+    assert a.layers[0].mixer == mixers.LinearAttentionSpec(3, 24, 40, 7.0)
+    assert a.layers[1].mixer == mixers.LatentAttentionSpec(2, 40, 24, 72, 40 ** -0.5, 50, None)
+    assert a.layers[2].mixer.kv_from == 1 and a.layers[2].mixer.window == 93 and a.layers[2].mlp is None
+    assert a.layers[3].mlp.ff == 130
+
+
+@pytest.mark.parametrize("change", [
+    lambda c: c.pop("width"),
+    lambda c: c.update(vocab=0),
+    lambda c: c.update(layers=[]),
+    lambda c: c["layers"][0].update(type="other"),
+    lambda c: c["layers"][0]["mixer"].pop("tau"),
+    lambda c: c["layers"][0]["mixer"].update(tau=0),
+    lambda c: c["layers"][0]["mixer"].update(heads=2.5),
+    lambda c: c["layers"][1]["mixer"]["mask"].update(size=0),
+    lambda c: c["layers"][0]["mlp"].update(kind="gated"),
+    lambda c: c["layers"][2]["mixer"].update(kv_from=0),           # not a latent layer
+    lambda c: c["layers"][2]["mixer"].update(kv_from=2),           # itself
+    lambda c: c["layers"][2]["mixer"].update(kv_from=4),           # later
+    lambda c: c["layers"][2]["mixer"].update(kv_rank=64),          # another rank
+])
+def test_bad_configs_are_refused(change):
+    c = copy.deepcopy(CONFIGS["mixed"])
+    change(c)
+    with pytest.raises(ValueError):
+        lositar.args_from_config(c)
+
+
+def test_registry_selects_by_config():
+    assert registry.resolve(CONFIGS["mixed"]).name == "lositar"
+    assert registry.resolve({"model_type": "qwen2"}).name == "llama"
+    assert set(registry.names()) == {"lositar", "llama"}
+    with pytest.raises(ValueError):
+        registry.resolve({"architecture": "Unheard"})
+
+
+def test_checkpoint_round_trip_and_shape_checks(tmp_path):
+    from safetensors.torch import save_file
+    cfg, w = CONFIGS["mixed"], weights("mixed")
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    model, got = checkpoint.load_model(tmp_path, CPU)
+    assert got == cfg and isinstance(model, hybrid.Model) and model.dtype == torch.bfloat16
+    model, _ = checkpoint.load_model(tmp_path, CPU, dtype="float32")
+    assert model.dtype == torch.float32 and torch.equal(model.embed_tokens[:203, :88], w["embed"].float())
+    assert registry.resolve(cfg).dtypes == ("bfloat16", "float32")
+    for name in ("l1.mix.dkv", "l0.mix.a2.b", "final.norm", "l0.norm2"):
+        with pytest.raises(ValueError, match=re.escape(name)):
+            lositar.build(cfg, {k: v for k, v in w.items() if k != name}, CPU)
+    for name in ("l1.mix.uk", "pos", "l3.mix.norm"):
+        bad = dict(w)
+        bad[name] = bad[name][..., :-1].contiguous()
+        with pytest.raises(ValueError, match=re.escape(name)):
+            lositar.build(cfg, bad, CPU)
+    bad = dict(w)
+    bad["l0.mix.a1"] = bad["l0.mix.a1"][:-1]
+    with pytest.raises(ValueError):
+        lositar.build(cfg, bad, CPU)
+    with pytest.raises(TypeError):
+        lositar.build(cfg, w, CPU, torch.float16)
+
+
+def test_padded_layout_reproduces_the_products():
+    """Products with the padded matrices, pads dropped, are the products with the checkpoint's."""
+    w = weights("mixed")
+    m = lositar.build(CONFIGS["mixed"], w, CPU, torch.float32)
+    h = torch.randn(5, 88)
+    hp = torch.nn.functional.pad(h, (0, m.layout.padded_width - 88))
+    g, gs = m.layers[0].mixer, CONFIGS["mixed"]["layers"][0]["mixer"]
+    y = hp @ g.proj.T
+    for name, off, d, dp in (("q", 0, 24, g.dkp), ("k", 1, 24, g.dkp), ("v", 2, 40, g.dvp), ("g", 3, 40, g.dvp)):
+        part = y[:, g.offsets[off]:g.offsets[off] + gs["heads"] * dp].reshape(5, gs["heads"], dp)
+        assert torch.allclose(part[..., :d].reshape(5, -1), h @ w[f"l0.mix.{name}"].float().T, atol=1e-4)
+        assert torch.equal(part[..., d:], torch.zeros(5, gs["heads"], dp - d))
+    a = y[:, g.offsets[4]:]
+    z = (a @ g.a2.T + g.a2_bias).reshape(5, 3, g.dkp)[..., :24].reshape(5, -1)
+    assert torch.allclose(z, h @ w["l0.mix.a1"].float().T @ w["l0.mix.a2"].float().T + w["l0.mix.a2.b"].float(), atol=1e-4)
+    o = torch.randn(5, 3, 40)
+    op = torch.zeros(5, g.o.shape[1])
+    op[:, :3 * g.dvp] = torch.nn.functional.pad(o, (0, g.dvp - 40)).reshape(5, -1)
+    assert torch.allclose((op @ g.o.T)[:, :88], o.reshape(5, -1) @ w["l0.mix.o"].float().T, atol=1e-4)
+    assert torch.allclose(m.layers[0].norm1[:88], 1 + w["l0.norm1"].float()) and not m.layers[0].norm1[88:].any()
+
+
+def test_caches_share_latents_and_refuse_a_rewound_state():
+    m = lositar.build(CONFIGS["mixed"], weights("mixed"), CPU)
+    c = cache.make_prompt_cache(m, capacity=10 ** 6)
+    assert len(c) == 5 and c[2] is c[1] and c[4] is not c[1]
+    assert c[0].capacity == 700                                   # no position beyond the learned ones
+    assert isinstance(c[0], cache.RecurrentState) and c[0].state.dtype == torch.float32
+    assert all(x.len_dev is c[0].len_dev for x in c)
+    c[0].offset = 5
+    c[0].state.fill_(1.0)
+    with pytest.raises(ValueError):
+        c[0].offset = 4
+    c.clear()
+    assert c[0].offset == 0 and not c[0].state.any() and int(c[0].len_dev) == 0
+
+
+def test_synthetic_config_is_a_config():
+    cfg = synth.lositar_config(width=64, layers=5, heads=2, dim=16, vdim=16, rank=64, ff=64, vocab=99, max_positions=128)
+    a = lositar.args_from_config(cfg)
+    assert [type(l.mixer).__name__[:6] for l in a.layers] == ["Latent", "Linear", "Latent", "Linear", "Latent"]
+    assert a.layers[2].mixer.kv_from == 0 and a.layers[4].mixer.kv_from is None
+    lositar.build(cfg, synth.make_lositar_weights(cfg), CPU)
+
+
+class FakeStream:
+    """Logits favour (last token + 1) mod 10; remembers what it was fed."""
+    made = 0
+
+    def __init__(self):
+        FakeStream.made += 1
+        self.fed = []
+
+    def clear(self):
+        self.fed = []
+
+    def feed(self, ids, want=None):
+        ids = list(ids)
+        self.fed += ids
+        rows = [len(ids) - 1] if want is None else list(want)
+        out = torch.zeros(len(rows), 10)
+        for r, w in enumerate(rows):
+            out[r, (ids[w] + 1) % 10] = len(self.fed)
+        return out
+
+    def pick(self, logits):
+        return int(logits[-1].argmax())
+
+    def greedy(self, token, n):
+        return [(token + 1 + i) % 10 for i in range(n)]
+
+
+def test_generate_feeds_portions_and_continues():
+    s = FakeStream()
+    s.fed = [9, 9]
+    assert generate.generate(None, [3, 1, 4, 1, 5], 4, prefill_step_size=2, stream=s) == [6, 7, 8, 9]
+    assert s.fed == [3, 1, 4, 1, 5]
+    assert generate.generate(None, [3], 1, stream=s) == [4] and generate.generate(None, [3], 0, stream=s) == []
+
+
+def test_trace_steps_reuse_finished_streams(tmp_path):
+    FakeStream.made = 0
+    r = trace.Requests(FakeStream)
+    y = trace.run_step(r, {"step": 0, "entries": [{"id": "a", "tokens": [1, 2, 3], "want": [0, 2]}, {"id": "b", "tokens": [7], "want": []}],
+                           "end": ["b"]})
+    assert y.shape == (2, 10) and y[0].argmax() == 2 and y[1].argmax() == 4 and set(r.live) == {"a"}
+    assert trace.run_step(r, {"step": 1, "entries": [{"id": "c", "tokens": [5]}], "end": []}) is None
+    assert FakeStream.made == 2 and r.live["c"].fed == [5]           # b's stream, cleared
+    y = trace.run_step(r, {"step": 2, "entries": [{"id": "a", "tokens": [4], "want": [0]}], "end": ["a", "c"]})
+    assert y.max() == 4 and not r.live and len(r.idle) == 2
+
+
+def test_trace_storage_types(tmp_path):
+    fams = {n: registry.resolve(c) for n, c in (("lositar", CONFIGS["mixed"]), ("llama", {}))}
+    assert trace.storage_type(fams["lositar"], "float32") == "float32"
+    assert trace.storage_type(fams["lositar"], "bfloat16") == "bfloat16"
+    assert trace.storage_type(fams["llama"], "bfloat16") == "float16"
+    assert trace.storage_type(fams["llama"], "float32") is None
+    (tmp_path / "config.json").write_text(json.dumps({"model_type": "qwen2"}))
+    assert trace.main(["--model", str(tmp_path), "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "8"],
+                      stdin=io.StringIO("")) == 3
+    assert os.access(os.path.join(ROOT, "bin", "trace_run"), os.X_OK)
+
+
+# ---- C ABI -------------------------------------------------------------------------------------
+
+
+def test_hybrid_library_exports_every_declared_symbol():
+    text = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "hybrid_mi355x.h")).read(), flags=re.S)
+    names = set(re.findall(r"\b(hyb_[a-z0-9_]+)\s*\(", text))
+    lib = ctypes.CDLL(_lib.HYBRID_LIB_PATH)
+    assert names == set(_lib.HYBRID_SIGNATURES) and all(hasattr(lib, n) for n in names)
+    assert _lib.hybrid().hyb_abi_version() == 1
+    for rc in range(7):
+        assert len(_lib.hybrid().hyb_status_string(rc)) > 1
+
+
+def _buf():
+    b = (ctypes.c_char * 4096)()
+    return b, (ctypes.addressof(b) + 15) & ~15
+
+
+def test_hybrid_argument_errors_are_detected_on_the_host():
+    L = _lib.hybrid()
+    keep, p = _buf()
+    assert L.hyb_embed(0, p, p, 1.0, p, 4, p, p, None, 1, 64, 8, None) == 1
+    assert L.hyb_embed(7, p, p, 1.0, p, 4, p, p, p, 1, 64, 8, None) == 4
+    assert L.hyb_embed(0, p, p, 1.0, p, 4, p, p, p, 1, 63, 8, None) == 2
+    assert L.hyb_norm_rows(0, p, None, p, 1e-5, p, None, 1, 64, 65, None) == 2
+    assert L.hyb_norm_rows(0, p + 4, None, p, 1e-5, p, None, 1, 64, 64, None) == 3
+
+    def dense(**kw):
+        d = dict(x=p, w=p, out=p, ldx=64, ldo=64, dtype=0, M=1, N=64, K=64, epilogue=0, form=-1)
+        d.update(kw)
+        return L.hyb_dense(ctypes.byref(_lib.HybDenseArgs(**d)), None)
+    assert dense(x=None) == 1 and dense(dtype=2) == 4 and dense(epilogue=5) == 4
+    assert dense(M=0) == 2 and dense(N=40) == 2 and dense(K=96) == 2 and dense(ldx=32) == 2 and dense(ldo=32) == 2
+    assert dense(w=p + 2) == 3
+    assert dense(M=5, norm_w=p, norm_d=64) == 4                  # the norm is part of the few-row form only
+    assert dense(M=65, form=1) == 4 and dense(M=5, form=0) == 4 and dense(norm_w=p, norm_d=64, form=2) == 4
+    assert dense(norm_w=p, norm_d=65) == 2
+    assert dense(epilogue=4, ldo=64) == 2 and dense(epilogue=4, ldo=128, bias=p) == 2
+    assert L.hyb_dense_form(0, 1, 64, 1, 0) == 0 and L.hyb_dense_form(0, 5, 64, 0, 0) == 1
+    assert L.hyb_dense_form(0, 65, 64, 0, 0) == 2 and L.hyb_dense_form(0, 2, 64, 0, 1) == 2
+    assert L.hyb_dense_form(1, 4, 1 << 16, 1, 0) == -1
+
+    def gla_call(fn, **kw):
+        d = dict(x=p, a2=p, a2_bias=p, z=p, norm_w=p, state=p, out=p, workspace=p, workspace_bytes=1 << 30, ldx=256, ldo=64,
+                 dtype=0, R=64, H=1, dkp=16, dvp=16, rp=64, dv_true=16, tau=1.0)
+        d.update(kw)
+        return getattr(L, fn)(ctypes.byref(_lib.HybGlaArgs(**d)), None)
+    for fn in ("hyb_gla_step", "hyb_gla_chunks"):
+        assert gla_call(fn, state=None) == 1 and gla_call(fn, dkp=24) == 2 and gla_call(fn, dvp=528) == 2
+        assert gla_call(fn, dv_true=17) == 2 and gla_call(fn, tau=0.0) == 2 and gla_call(fn, off_v=3) == 3
+    assert gla_call("hyb_gla_step", a2=None) == 1 and gla_call("hyb_gla_step", rp=4) == 2
+    assert gla_call("hyb_gla_chunks", z=None) == 1 and gla_call("hyb_gla_chunks", R=63) == 2
+    assert gla_call("hyb_gla_chunks", workspace_bytes=64) == 5
+    assert L.hyb_gla_chunk_workspace_bytes(65, 2, 16, 32) == 2 * 2 * (64 * 64 + 16 * 32 + 16) * 4
+
+    assert L.hyb_latent_append(0, p, 64, p, 1e-5, p, 8, p, p, 1, 60, 60, None) == 2
+    assert L.hyb_latent_append(0, p, 64, p, 1e-5, None, 8, p, p, 1, 64, 64, None) == 1
+    assert [L.hyb_latent_rank_supported(r) for r in (64, 96, 512, 576, 768, 1024, 1088)] == [1, 0, 1, 0, 1, 1, 0]
+
+    def decode(**kw):
+        d = dict(q=p, cache=p, uk=p, uv=p, gate=p, out=p, len_dev=p, workspace=p, workspace_bytes=1 << 30, ldq=64, ldg=64,
+                 ldo=64, cap=128, dtype=0, R=1, H=1, dp=32, dvp=16, rank=64, window=8, scale=1.0)
+        d.update(kw)
+        return L.hyb_latent_decode(ctypes.byref(_lib.HybLatentDecodeArgs(**d)), None)
+    assert decode(uv=None) == 1 and decode(R=65) == 2 and decode(rank=96) == 2 and decode(window=0) == 2 and decode(ldq=16) == 2
+    assert decode(cache=p + 2) == 3 and decode(workspace_bytes=16) == 5
+    assert decode(append=p) == 1 and decode(append=p, append_norm=p, ldappend=32, rank_true=64) == 2
+
+    def window(**kw):
+        d = dict(q=p, k=p, vt=p, gate=p, out=p, len_dev=p, ldq=64, ldk=64, ldv=128, ldg=64, ldo=64, dtype=0, R=64, H=1, dp=32,
+                 dvp=16, window=8, back=7, scale=1.0)
+        d.update(kw)
+        return L.hyb_window_attention(ctypes.byref(_lib.HybWindowArgs(**d)), None)
+    assert window(k=None) == 1 and window(dp=48) == 2 and window(dvp=272) == 2 and window(back=8) == 2 and window(ldv=64) == 2
+    assert window(ldv=100) == 2 and window(vt=p + 2) == 3
+    assert L.hyb_argmax_rows_f32(p, 10, 1, 11, p, p, 1 << 20, None) == 2
+    assert L.hyb_argmax_rows_f32(p, 10, 1, 10, p, None, 0, None) == 5
+    assert L.hyb_token_advance(p, p, p, None, 4, None) == 1 and L.hyb_advance_len(p, p, 0, None) == 2
+    del keep
