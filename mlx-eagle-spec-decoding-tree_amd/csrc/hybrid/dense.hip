@@ -258,7 +258,8 @@ __global__ __launch_bounds__(512) void dense_skinny_kernel(DenseP p) {
 }
 
 // Form 3, many rows: BM x BN output block, four waves 2 x 2, 128 bytes of K per step through LDS
-// (double buffered, 16-byte chunks xored with the row so that reads spread over the banks).
+// (double buffered, 16-byte chunks xored with the row so that reads spread over the banks) and two more
+// steps on their way in registers.
 // TRANS: the block is stored transposed, out[n][m].
 template <typename T, int BM, int BN, bool TRANS>
 __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(DenseP p, int tiles_m, int tiles_n) {
@@ -290,19 +291,22 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(DenseP p, int tiles_
     const int n = n0 + srow + 32 * i;
     wp[i] = reinterpret_cast<const T*>(p.w) + (size_t)(n < p.N ? n : p.N - 1) * p.K + chunk * EPC;
   }
-  u32x4_t xr[TM], wr[TN];
-  auto fetch = [&](int k) {
+  // Two steps of K in registers on their way to LDS.  Fetches are unconditional (the last steps repeat),
+  // so that a wait for the older step never has to assume that the newer one was not issued.
+  u32x4_t xr[2][TM], wr[2][TN];
+  auto fetch = [&](int set, int k) {
+    k = k < p.K ? k : p.K - BK;
 #pragma unroll
-    for (int i = 0; i < TM; ++i) xr[i] = *reinterpret_cast<const u32x4_t*>(xp[i] + k);
+    for (int i = 0; i < TM; ++i) xr[set][i] = *reinterpret_cast<const u32x4_t*>(xp[i] + k);
 #pragma unroll
-    for (int i = 0; i < TN; ++i) wr[i] = *reinterpret_cast<const u32x4_t*>(wp[i] + k);
+    for (int i = 0; i < TN; ++i) wr[set][i] = *reinterpret_cast<const u32x4_t*>(wp[i] + k);
   };
   const int spos = srow * 128 + ((chunk ^ (srow & 7)) << 4);
-  auto put = [&](int buf) {
+  auto put = [&](int buf, int set) {
 #pragma unroll
-    for (int i = 0; i < TM; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][spos + i * 32 * 128]) = xr[i];
+    for (int i = 0; i < TM; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][spos + i * 32 * 128]) = xr[set][i];
 #pragma unroll
-    for (int i = 0; i < TN; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][BM * 128 + spos + i * 32 * 128]) = wr[i];
+    for (int i = 0; i < TN; ++i) *reinterpret_cast<u32x4_t*>(&lds[buf][BM * 128 + spos + i * 32 * 128]) = wr[set][i];
   };
   const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * (BN / 2);
   auto frag = [&](const unsigned char* base, int row, int s) {
@@ -322,13 +326,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(DenseP p, int tiles_
 #pragma unroll
     for (int b = 0; b < TN; ++b) acc[a][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
-  fetch(0);
-  put(0);
-  __syncthreads();
-  int buf = 0;
-  for (int k = 0; k < p.K; k += BK) {
-    const bool more = k + BK < p.K;
-    if (more) fetch(k + BK);
+  auto compute = [&](int buf) {
     const unsigned char* xl = lds[buf];
     const unsigned char* wl = lds[buf] + BM * 128;
 #pragma unroll
@@ -343,10 +341,22 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(DenseP p, int tiles_
 #pragma unroll
         for (int b = 0; b < TN; ++b) acc[a][b] = TRANS ? mma(xf[a], wf[b], acc[a][b]) : mma(wf[b], xf[a], acc[a][b]);
     }
-    if (more) {
-      put(buf ^ 1);
-      __syncthreads();
-      buf ^= 1;
+  };
+  fetch(0, 0);
+  fetch(1, BK);
+  put(0, 0);
+  __syncthreads();
+  for (int k = 0; k < p.K; k += 2 * BK) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {          // step k + u BK is in LDS buffer u
+      const int kk = k + u * BK;
+      if (kk >= p.K) break;
+      fetch(u, kk + 2 * BK);
+      compute(u);
+      if (kk + BK < p.K) {
+        put(u ^ 1, u ^ 1);
+        __syncthreads();
+      }
     }
   }
 #pragma unroll
