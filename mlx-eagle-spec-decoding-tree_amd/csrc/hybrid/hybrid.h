@@ -116,7 +116,7 @@ __device__ inline Frag<float> as_frag(const Wide8& w) {
   for (int e = 0; e < 8; ++e) f.set(e, w.v[e]);
   return f;
 }
-// c += A B with A fp32 / with B fp32
+// c += A B with A given in fp32
 __device__ inline f32x4_t mma_wide_a(const Wide8& a, const Frag<bf16_t>& b, f32x4_t c) {
   Frag<bf16_t> hi, lo;
   split(a, hi, lo);
